@@ -3,6 +3,10 @@
 // the router wrote: a pair streams its expert's gate and up rows against the token's row and applies silu(gate) * up;
 // a token's output row is the weighted sum over its pairs of the expert's down rows against the pair's hidden row.
 // Sums are 32-bit; the hidden row is rounded once to the activations' type; the output is float32.
+//
+// Beside the experts that have matrices there may be identity experts: choices from `experts` on, whose output is the token's
+// row itself.  And there may be a shared expert that every token uses, weighted by a gate of one number a token: its
+// products are made inside the same two kernels (steps of few tokens), or its output comes ready made.
 #include "common.hpp"
 
 using namespace lsa;
@@ -86,12 +90,17 @@ __global__ __launch_bounds__(256) void route_logits_kernel(const float* __restri
 }
 
 // One wavefront per token: the `top` largest of the token's float32 logits (the lowest index among equal ones) and
-// their softmax.  The logits themselves are a float32 matrix product made before this kernel.  A lane keeps the logits
+// their softmax.  The logits themselves are a float32 matrix product made before this kernel, rows of `stride` numbers.
+// scoring 0: that; 1: sigmoid(logits) are scores, choice values and weights; 2: the scores are the softmax over all experts,
+// the choice values scores + correction, the weights the chosen scores divided by (their sum + 1e-20), times weight_scale.
+// gate_out (or nullptr): sigmoid of the logit behind the experts', a gate of one number a token.  A lane keeps the logits
 // of experts lane, lane + 64, ... in LDS (its own entries only: nothing crosses lanes through LDS), and every lane ends
 // each round with the same (best, where).
 __global__ __launch_bounds__(256) void route_top_kernel(const float* __restrict__ all_logits, int experts, int top,
                                                         int* __restrict__ chosen, float* __restrict__ weights, int n_tokens,
-                                                        int sigmoid_scores, int groups, int keep, const float* __restrict__ bias) {
+                                                        int scoring, int groups, int keep, const float* __restrict__ bias,
+                                                        const float* __restrict__ correction, float weight_scale, int stride,
+                                                        float* __restrict__ gate_out) {
     extern __shared__ float lds[];
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int t = blockIdx.x * (blockDim.x >> 6) + wave;
@@ -99,13 +108,26 @@ __global__ __launch_bounds__(256) void route_top_kernel(const float* __restrict_
     // (two arrays a wavefront: the values the choice is made among, and, for sigmoid scores, the scores themselves)
     float* logits = lds + (size_t)wave * 2 * experts;
     float* scores = logits + experts;
+    const bool sigmoid_scores = scoring == 1;
+    if (gate_out && lane == 0) gate_out[t] = 1.f / (1.f + expf(-all_logits[(size_t)t * stride + experts]));
+    float most = 0.f, all = 1.f;
+    if (scoring == 2) {                                        // the softmax over all experts
+        most = NEG_INF;
+        for (int e = lane; e < experts; e += 64) most = fmaxf(most, all_logits[(size_t)t * stride + e] + (bias ? bias[e] : 0.f));
+        most = wave_max(most);
+        all = 0.f;
+        for (int e = lane; e < experts; e += 64) all += expf(all_logits[(size_t)t * stride + e] + (bias ? bias[e] : 0.f) - most);
+        all = wave_sum(all);
+    }
     for (int e = lane; e < experts; e += 64) {
-        float v = all_logits[(size_t)t * experts + e];
+        float v = all_logits[(size_t)t * stride + e];
         if (bias) v += bias[e];                            // (a bias per expert joins the logits)
         if (sigmoid_scores) v = 1.f / (1.f + expf(-v));
-        logits[e] = v;
+        if (scoring == 2) v = expf(v - most) / all;
         scores[e] = v;
+        logits[e] = correction ? v + correction[e] : v;
     }
+    __builtin_amdgcn_wave_barrier();
     if (sigmoid_scores && groups > 1) {
         // A group's score is the sum of its two largest scores; the `keep` best groups stay (the first of equal ones),
         // the experts of the others cannot be chosen.  Lane g (and g + 64, ...) scores group g; entries of other lanes
@@ -151,7 +173,9 @@ __global__ __launch_bounds__(256) void route_top_kernel(const float* __restrict_
         }
         if (where >= experts) where = k < experts ? k : 0;        // (only if every logit left is NaN or -inf)
         if (k == 0) largest = best;
-        const float weight = sigmoid_scores ? best : expf(best - largest);
+        float weight = sigmoid_scores ? best : expf(best - largest);
+        // (a score stands in the entries of the lane that owns the expert; the wavefront's LDS operations keep their order)
+        if (scoring == 2) weight = scores[where];
         total += weight;
         if (lane == 0) {
             chosen[(size_t)t * top + k] = where;
@@ -159,18 +183,28 @@ __global__ __launch_bounds__(256) void route_top_kernel(const float* __restrict_
         }
         if ((where & 63) == lane) logits[where] = NEG_INF;
     }
-    if (lane == 0 && !sigmoid_scores)
+    if (lane == 0 && scoring == 0)
         for (int k = 0; k < top; ++k) weights[(size_t)t * top + k] /= total;         // (its own writes)
+    if (lane == 0 && scoring == 2)
+        for (int k = 0; k < top; ++k) weights[(size_t)t * top + k] = weights[(size_t)t * top + k] / (total + 1e-20f) * weight_scale;
 }
 
-// grid (pairs, blocks of hidden columns): hidden[pair][f] = silu(G[f] . x) * (U[f] . x) for the pair's expert.
+// grid (pairs, blocks of hidden columns): hidden[pair][f] = silu(G[f] . x) * (U[f] . x) for the pair's expert.  With a shared
+// expert a token has one more pair, the last: the shared expert's matrices and its own hidden row [tokens][shared_inter].
+// Pairs of identity experts (choices from `experts` on, where `identity`) have nothing to multiply.
 template <typename T>
 __global__ __launch_bounds__(256) void experts_gate_up_kernel(const T* __restrict__ x, const T* __restrict__ gate_up,
                                                               const int* __restrict__ chosen, T* __restrict__ hidden, int top,
                                                               int inter, int width, int experts, int columns_per_block, bool in_lds,
-                                                              float limit) {
+                                                              float limit, int identity, const T* __restrict__ shared_gate_up,
+                                                              T* __restrict__ shared_hidden, int shared_inter) {
     extern __shared__ __align__(16) unsigned char lds_bytes[];
-    const int pair = blockIdx.x, t = pair / top;
+    const int slots = top + (shared_gate_up ? 1 : 0), t = blockIdx.x / slots, slot = blockIdx.x - t * slots;
+    const bool shared = slot == top;
+    const int pair = t * top + slot;
+    int expert = shared ? 0 : chosen[pair];
+    if (identity && expert >= experts) return;               // (the whole workgroup)
+    if ((int)blockIdx.y * columns_per_block >= (shared ? shared_inter : inter)) return;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, waves = blockDim.x >> 6;
     const T* x_lds = x + (size_t)t * width;                  // (a row too long for LDS is read where it lies)
     if (in_lds) {
@@ -179,25 +213,37 @@ __global__ __launch_bounds__(256) void experts_gate_up_kernel(const T* __restric
         __syncthreads();
         x_lds = staged;
     }
-    int expert = chosen[pair];
     expert = expert < 0 ? 0 : expert >= experts ? experts - 1 : expert;
-    const T* base = gate_up + (size_t)expert * 2 * inter * width;
+    const T* base = shared ? shared_gate_up : gate_up + (size_t)expert * 2 * inter * width;
+    T* result = shared ? shared_hidden + (size_t)t * shared_inter : hidden + (size_t)pair * inter;
+    if (shared) inter = shared_inter;
     const int f0 = blockIdx.y * columns_per_block, f1 = min(inter, f0 + columns_per_block);
     for (int f = f0 + wave; f < f1; f += waves) {
         float g, u;
         wave_dot2(base + (size_t)f * width, base + (size_t)(inter + f) * width, x_lds, width, lane, g, u);
-        if (lane == 0) hidden[(size_t)pair * inter + f] = (T)gated_activation(g, u, limit);
+        if (lane == 0) result[f] = (T)gated_activation(g, u, limit);
     }
 }
 
 // grid (tokens, blocks of output columns): out[t][c] = sum_s weights[t][s] * (D_s[c] . hidden[t * top + s]).
 // A wavefront owns a column: every lane adds up its share of all `top` dot products, weighted, and the lanes' sums meet
-// once at the end; the loads of all pairs' rows are independent of one another.
+// once at the end; the loads of all pairs' rows are independent of one another.  Added to that: the token's row x times the
+// weights of its identity experts (choices from `experts` on, where x is given), and the shared expert's output times the
+// token's gate: shared_y ready made, or shared_down[c] . shared_hidden[t].
+template <typename T> struct BesideExperts {
+    const T* x;                     // [tokens][width], or nullptr: no identity experts
+    const float* gate;              // [tokens]: what the shared expert's output is multiplied by, or nullptr: no shared expert
+    const T* y;                     // [tokens][width]: its output, or nullptr: the two below
+    const T* down;                  // [width][inter]
+    const T* hidden;                // [tokens][inter]
+    int inter;
+};
+
 template <typename T>
 __global__ __launch_bounds__(256) void experts_down_kernel(const T* __restrict__ hidden, const T* __restrict__ down,
                                                            const int* __restrict__ chosen, const float* __restrict__ weights,
                                                            float* __restrict__ out, int top, int inter, int width, int experts,
-                                                           int columns_per_block, bool in_lds) {
+                                                           int columns_per_block, bool in_lds, BesideExperts<T> beside) {
     extern __shared__ __align__(16) unsigned char lds_bytes[];
     constexpr int V = Elem<T>::kVec;
     const int t = blockIdx.x;
@@ -214,11 +260,20 @@ __global__ __launch_bounds__(256) void experts_down_kernel(const T* __restrict__
     constexpr int MOST = 128;
     __shared__ int expert_of[MOST];
     __shared__ float weight_of[MOST];
+    __shared__ float identity_weight;
     for (int s = threadIdx.x; s < min(top, MOST); s += blockDim.x) {
         const int expert = chosen[(size_t)t * top + s];
-        expert_of[s] = expert < 0 ? 0 : expert >= experts ? experts - 1 : expert;
+        expert_of[s] = beside.x && expert >= experts ? -1 : expert < 0 ? 0 : expert >= experts ? experts - 1 : expert;
         weight_of[s] = weights[(size_t)t * top + s];
     }
+    if (threadIdx.x == 0 && beside.x) {
+        float total = 0.f;
+        for (int s = 0; s < top; ++s)
+            if (chosen[(size_t)t * top + s] >= experts) total += weights[(size_t)t * top + s];
+        identity_weight = total;
+    }
+    const float gate = beside.gate ? beside.gate[t] : 0.f;
+    const bool shared_vectors = beside.inter % V == 0 && ((reinterpret_cast<size_t>(beside.down) | reinterpret_cast<size_t>(beside.hidden)) & 15) == 0;
     __syncthreads();
     const int c0 = blockIdx.y * columns_per_block, c1 = min(width, c0 + columns_per_block);
     for (int c = c0 + wave; c < c1; c += waves) {
@@ -229,6 +284,7 @@ __global__ __launch_bounds__(256) void experts_down_kernel(const T* __restrict__
             const int pieces = inter / V, all = top * pieces;
             for (int p = lane; p < all; p += 64) {
                 const int s = p / pieces, i = (p - s * pieces) * V;
+                if (expert_of[s] < 0) continue;          // (an identity expert)
                 const Vec16<T> a = load_vec16(down + ((size_t)expert_of[s] * width + c) * inter + i);
                 const Vec16<T> b = *reinterpret_cast<const Vec16<T>*>(h_lds + (size_t)s * inter + i);
                 float part = 0.f;
@@ -239,6 +295,7 @@ __global__ __launch_bounds__(256) void experts_down_kernel(const T* __restrict__
         } else {
             for (int s = 0; s < top; ++s) {
                 int expert = chosen[(size_t)t * top + s];
+                if (beside.x && expert >= experts) continue;
                 expert = expert < 0 ? 0 : expert >= experts ? experts - 1 : expert;
                 const T* row = down + ((size_t)expert * width + c) * inter;
                 const T* h = h_lds + (size_t)s * inter;
@@ -247,8 +304,27 @@ __global__ __launch_bounds__(256) void experts_down_kernel(const T* __restrict__
                 acc += weights[(size_t)t * top + s] * part;
             }
         }
+        if (beside.down) {
+            const T* row = beside.down + (size_t)c * beside.inter;
+            const T* h = beside.hidden + (size_t)t * beside.inter;
+            float part = 0.f;
+            if (shared_vectors) {
+                for (int i = lane * V; i < beside.inter; i += 64 * V) {
+                    const Vec16<T> a = load_vec16(row + i), b = load_vec16(h + i);
+#pragma unroll
+                    for (int k = 0; k < V; ++k) part += (float)a.v[k] * (float)b.v[k];
+                }
+            } else {
+                for (int i = lane; i < beside.inter; i += 64) part += (float)row[i] * (float)h[i];
+            }
+            acc += gate * part;
+        }
         acc = wave_sum(acc);
-        if (lane == 0) out[(size_t)t * width + c] = acc;
+        if (lane == 0) {
+            if (beside.y) acc += gate * (float)beside.y[(size_t)t * width + c];
+            if (beside.x) acc += identity_weight * (float)beside.x[(size_t)t * width + c];
+            out[(size_t)t * width + c] = acc;
+        }
     }
 }
 
@@ -258,41 +334,51 @@ LSA_EXPORT int lsa_route_logits(const float* x, const float* router, float* logi
     LSA_LAUNCH_CHECK();
 }
 
-// sigmoid_scores: the choice is made among sigmoid(logits), which are the weights as they are; groups > 1: only the
-// experts of the `keep` best of `groups` equal groups of neighbours can be chosen (at most 64 groups).
-LSA_EXPORT int lsa_route_top(const float* logits, int experts, int top, int* chosen, float* weights, int n, int sigmoid_scores,
-                             int groups, int keep, const float* bias, hipStream_t stream) {
+// scoring 1: the choice is made among sigmoid(logits), which are the weights as they are; groups > 1: only the
+// experts of the `keep` best of `groups` equal groups of neighbours can be chosen (at most 64 groups).  scoring 2: see the kernel.
+LSA_EXPORT int lsa_route_top(const float* logits, int experts, int top, int* chosen, float* weights, int n, int scoring,
+                             int groups, int keep, const float* bias, const float* correction, float weight_scale, int stride, float* gate_out,
+                             hipStream_t stream) {
     if (n <= 0) return 0;
+    const bool sigmoid_scores = scoring == 1;
+    if (scoring < 0 || scoring > 2 || (correction != nullptr && scoring != 2) || stride < experts + (gate_out ? 1 : 0)) return -1;
     if (top < 1 || top > experts || (size_t)experts * 32 > 60000) return -1;
     if (groups > 1 && (!sigmoid_scores || groups > 64 || experts % groups || keep < 1 || keep > groups || top > keep * (experts / groups))) return -1;
     route_top_kernel<<<(n + 3) / 4, 256, (size_t)experts * 8 * sizeof(float), stream>>>(logits, experts, top, chosen, weights, n,
-                                                                                       sigmoid_scores, groups, keep, bias);
+                                                                                       scoring, groups, keep, bias, correction, weight_scale, stride, gate_out);
     LSA_LAUNCH_CHECK();
 }
 
 LSA_EXPORT int lsa_experts_gate_up(int code, const void* x, const void* gate_up, const int* chosen, void* hidden, int n, int top,
-                                   int inter, int width, int experts, float limit, hipStream_t stream) {
+                                   int inter, int width, int experts, float limit, int identity, const void* shared_gate_up,
+                                   void* shared_hidden, int shared_inter, hipStream_t stream) {
     if (n <= 0) return 0;
+    if (shared_gate_up != nullptr && (shared_hidden == nullptr || shared_inter < 1)) return -1;
+    const int most_inter = shared_gate_up && shared_inter > inter ? shared_inter : inter;
     size_t lds = (size_t)width * (code ? 2 : 4);
     const bool in_lds = lds <= 64000;
     if (!in_lds) lds = 0;
     const int columns = 16;
-    dim3 grid(n * top, (inter + columns - 1) / columns);
-    if (code) experts_gate_up_kernel<bf16_t><<<grid, 256, lds, stream>>>((const bf16_t*)x, (const bf16_t*)gate_up, chosen, (bf16_t*)hidden, top, inter, width, experts, columns, in_lds, limit);
-    else experts_gate_up_kernel<float><<<grid, 256, lds, stream>>>((const float*)x, (const float*)gate_up, chosen, (float*)hidden, top, inter, width, experts, columns, in_lds, limit);
+    dim3 grid(n * (top + (shared_gate_up ? 1 : 0)), (most_inter + columns - 1) / columns);
+    if (code) experts_gate_up_kernel<bf16_t><<<grid, 256, lds, stream>>>((const bf16_t*)x, (const bf16_t*)gate_up, chosen, (bf16_t*)hidden, top, inter, width, experts, columns, in_lds, limit, identity, (const bf16_t*)shared_gate_up, (bf16_t*)shared_hidden, shared_inter);
+    else experts_gate_up_kernel<float><<<grid, 256, lds, stream>>>((const float*)x, (const float*)gate_up, chosen, (float*)hidden, top, inter, width, experts, columns, in_lds, limit, identity, (const float*)shared_gate_up, (float*)shared_hidden, shared_inter);
     LSA_LAUNCH_CHECK();
 }
 
 LSA_EXPORT int lsa_experts_down(int code, const void* hidden, const void* down, const int* chosen, const float* weights, float* out,
-                                int n, int top, int inter, int width, int experts, hipStream_t stream) {
+                                int n, int top, int inter, int width, int experts, const void* x, const float* shared_gate, const void* shared_y,
+                                const void* shared_down, const void* shared_hidden, int shared_inter, hipStream_t stream) {
     if (n <= 0) return 0;
+    if ((shared_gate != nullptr) != (shared_y != nullptr || shared_down != nullptr) || (shared_down != nullptr && shared_hidden == nullptr)) return -1;
     // (a block takes four columns: staging the token's hidden rows in LDS would cost as much as it reads of the weights)
     const size_t lds = 0;
     const bool in_lds = false;
     const int columns = 4;
     dim3 grid(n, (width + columns - 1) / columns);
-    if (code) experts_down_kernel<bf16_t><<<grid, 256, lds, stream>>>((const bf16_t*)hidden, (const bf16_t*)down, chosen, weights, out, top, inter, width, experts, columns, in_lds);
-    else experts_down_kernel<float><<<grid, 256, lds, stream>>>((const float*)hidden, (const float*)down, chosen, weights, out, top, inter, width, experts, columns, in_lds);
+#define LSA_BESIDE(T) BesideExperts<T>{(const T*)x, shared_gate, (const T*)shared_y, (const T*)shared_down, (const T*)shared_hidden, shared_inter}
+    if (code) experts_down_kernel<bf16_t><<<grid, 256, lds, stream>>>((const bf16_t*)hidden, (const bf16_t*)down, chosen, weights, out, top, inter, width, experts, columns, in_lds, LSA_BESIDE(bf16_t));
+    else experts_down_kernel<float><<<grid, 256, lds, stream>>>((const float*)hidden, (const float*)down, chosen, weights, out, top, inter, width, experts, columns, in_lds, LSA_BESIDE(float));
+#undef LSA_BESIDE
     LSA_LAUNCH_CHECK();
 }
 
@@ -464,10 +550,28 @@ __global__ __launch_bounds__(256) void experts_tile_kernel(const bf16_t* __restr
         }
 }
 
-// out[t][c] = sum_s weights[t][s] * y[t * top + s][c]
+// out[t][c] = sum_s weights[t][s] * y[t * top + s][c]; with `beside`: identity experts (choices from `experts` on) put the token's
+// row in place of y, and the shared expert's output joins times the token's gate.
 __global__ __launch_bounds__(256) void experts_combine_kernel(const float* __restrict__ y, const float* __restrict__ weights,
-                                                              float* __restrict__ out, int top, int width) {
+                                                              float* __restrict__ out, int top, int width, const int* __restrict__ chosen,
+                                                              int experts, BesideExperts<bf16_t> beside) {
     const int t = blockIdx.x;
+    if (beside.x || beside.gate) {
+        const float gate = beside.gate ? beside.gate[t] : 0.f;
+        float identity_weight = 0.f;
+        if (beside.x)
+            for (int s = 0; s < top; ++s)
+                if (chosen[(size_t)t * top + s] >= experts) identity_weight += weights[(size_t)t * top + s];
+        for (int c = threadIdx.x; c < width; c += blockDim.x) {
+            float acc = 0.f;
+            for (int s = 0; s < top; ++s)
+                if (!beside.x || chosen[(size_t)t * top + s] < experts) acc += weights[(size_t)t * top + s] * y[((size_t)t * top + s) * width + c];
+            if (beside.gate) acc += gate * (float)beside.y[(size_t)t * width + c];
+            if (beside.x) acc += identity_weight * (float)beside.x[(size_t)t * width + c];
+            out[(size_t)t * width + c] = acc;
+        }
+        return;
+    }
     for (int c = threadIdx.x; c < width; c += blockDim.x) {
         float acc = 0.f;
         for (int s = 0; s < top; ++s) acc += weights[(size_t)t * top + s] * y[((size_t)t * top + s) * width + c];
@@ -481,8 +585,10 @@ LSA_EXPORT int lsa_experts_tile_rows() { return TILE_M; }
 // Scratch: sorted [max_tiles * 64] and tile_expert [max_tiles] ints, y [pairs, width] floats; max_tiles >= ceil(pairs / 64) + experts.
 LSA_EXPORT int lsa_experts_tiled(const void* x, const void* gate_up, const void* down, const int* chosen, const float* weights,
                                  void* hidden, float* y, float* out, int* sorted, int* tile_expert, int max_tiles, int n, int top,
-                                 int inter, int width, int experts, float limit, hipStream_t stream) {
+                                 int inter, int width, int experts, float limit, int identity, const float* shared_gate, const void* shared_y,
+                                 hipStream_t stream) {
     if (n <= 0) return 0;
+    if ((shared_gate != nullptr) != (shared_y != nullptr)) return -1;
     const int pairs = n * top;
     if (width % 32 || inter % 32 || max_tiles < (pairs + TILE_M - 1) / TILE_M + experts || (size_t)experts * 8 > 60000) return -1;
     experts_sort_kernel<<<1, 1024, (size_t)experts * 2 * sizeof(int), stream>>>(chosen, pairs, experts, sorted, tile_expert, max_tiles);
@@ -505,6 +611,7 @@ LSA_EXPORT int lsa_experts_tiled(const void* x, const void* gate_up, const void*
         else LSA_TILES(32, 4);
     }
 #undef LSA_TILES
-    experts_combine_kernel<<<n, 256, 0, stream>>>(y, weights, out, top, width);
+    experts_combine_kernel<<<n, 256, 0, stream>>>(y, weights, out, top, width, chosen, experts,
+                                                 BesideExperts<bf16_t>{identity ? xb : nullptr, shared_gate, (const bf16_t*)shared_y, nullptr, nullptr, 0});
     LSA_LAUNCH_CHECK();
 }

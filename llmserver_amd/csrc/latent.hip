@@ -1,18 +1,20 @@
 // Around attention over a shared low-rank latent: one row [latent, rotated key part, zeros] per token is the token's
 // key and, transposed, its value in a paged cache with one key-value head; a query head's row is
-// [its query mapped into the latent, its rotated part, zeros].  Rotation turns neighbouring dimensions (2i, 2i+1)
-// together by the token's angle i; norm, rotation and sigmoid are 32-bit, every result is rounded once.
+// [its query mapped into the latent, its rotated part, zeros].  Rotation turns neighbouring dimensions (2i, 2i+1), or
+// dimensions i and i + pairs, together by the token's angle i; norm, rotation and sigmoid are 32-bit, every result is rounded once.
 #include "common.hpp"
 
 using namespace lsa;
 
 // The rotated value of element e of a vector whose first 2 * pairs elements turn; cs = the token's [cos.., sin..].
+// halves: element i turns with element i + pairs; otherwise neighbours (2i, 2i + 1) turn together.
 template <typename T>
-__device__ inline float turned(const T* __restrict__ v, int e, const float* __restrict__ cs, int pairs) {
-    const int pair = e >> 1;
-    if (pair >= pairs) return (float)v[e];
-    const float u = (float)v[2 * pair], w = (float)v[2 * pair + 1], c = cs[pair], s = cs[pairs + pair];
-    return (e & 1) ? w * c + u * s : u * c - w * s;
+__device__ inline float turned(const T* __restrict__ v, int e, const float* __restrict__ cs, int pairs, int halves) {
+    if (e >= 2 * pairs) return (float)v[e];
+    const int pair = halves ? (e < pairs ? e : e - pairs) : e >> 1;
+    const bool second = halves ? e >= pairs : (e & 1);
+    const float u = (float)v[halves ? pair : 2 * pair], w = (float)v[halves ? pairs + pair : 2 * pair + 1], c = cs[pair], s = cs[pairs + pair];
+    return second ? w * c + u * s : u * c - w * s;
 }
 
 // grid (tokens, heads + 1, pieces of 64 of a row).  proj row: heads x [dim plain, rot_dim rotated] query dimensions, then
@@ -28,7 +30,7 @@ __global__ void latent_prepare_kernel(
     const float* __restrict__ norm_weight, float eps,
     const float* __restrict__ cos_sin, int pairs, T* __restrict__ keys, T* __restrict__ values, const int* __restrict__ table,
     int table_stride, const int* __restrict__ token_row, const int* __restrict__ positions, int page_size, T* __restrict__ out_q,
-    int heads, int dim, int rot_dim, int rank, int row_width, int write_cache, int n_tokens) {
+    int heads, int dim, int rot_dim, int rank, int row_width, int write_cache, int n_tokens, int halves) {
     __shared__ float scratch[16];
     __shared__ float partial[4][64];
     const int t = blockIdx.x, head = blockIdx.y;
@@ -42,7 +44,7 @@ __global__ void latent_prepare_kernel(
             for (int e = threadIdx.x; e < row_width; e += blockDim.x) {
                 float v = 0.f;
                 if (e < rank) v = (float)q_latent[((size_t)head * n_tokens + t) * rank + e];
-                else if (e < rank + rot_dim) v = turned(qh + dim, e - rank, cs, pairs);
+                else if (e < rank + rot_dim) v = turned(qh + dim, e - rank, cs, pairs, halves);
                 out_q[((size_t)t * heads + head) * row_width + e] = (T)v;
             }
             return;
@@ -68,7 +70,7 @@ __global__ void latent_prepare_kernel(
         v = 0.f;
         for (int w = 0; w < waves; ++w) v += partial[w][lane];
         if (e >= row_width) return;
-        if (e >= rank) v = e < rank + rot_dim ? turned(qh + dim, e - rank, cs, pairs) : 0.f;
+        if (e >= rank) v = e < rank + rot_dim ? turned(qh + dim, e - rank, cs, pairs, halves) : 0.f;
         out_q[((size_t)t * heads + head) * row_width + e] = (T)v;
         return;
     }
@@ -88,7 +90,7 @@ __global__ void latent_prepare_kernel(
     for (int e = threadIdx.x; e < row_width; e += blockDim.x) {
         float v = 0.f;
         if (e < rank) v = (float)down[e] * inv * norm_weight[e];
-        else if (e < rank + rot_dim) v = turned(down + rank, e - rank, cs, pairs);
+        else if (e < rank + rot_dim) v = turned(down + rank, e - rank, cs, pairs, halves);
         key[e] = (T)v;
         value[(size_t)e * page_size] = (T)v;
     }
@@ -147,14 +149,14 @@ LSA_EXPORT int lsa_latent_prepare(int code, const void* proj, long proj_stride, 
                                   const float* norm_weight, float eps,
                                   const float* cos_sin, int pairs, void* keys, void* values, const int* table, int table_stride,
                                   const int* token_row, const int* positions, int page_size, void* out_q, int heads, int dim, int rot_dim,
-                                  int rank, int row_width, int write_cache, int n_tokens, hipStream_t stream) {
+                                  int rank, int row_width, int write_cache, int n_tokens, int halves, hipStream_t stream) {
     if (n_tokens <= 0) return 0;
     if (rank + rot_dim > row_width || 2 * pairs > rot_dim || page_size <= 0 || (q_latent == nullptr) == (up_keys == nullptr)) return -1;
     // (256 threads where the product is made here and for the cache row's norm; the copy alone needs a wavefront a piece)
     dim3 grid(n_tokens, heads + 1, up_keys ? (row_width + 63) / 64 : 1);
 #define LSA_LAUNCH(T) latent_prepare_kernel<T><<<grid, 256, 0, stream>>>((const T*)proj, proj_stride, (const T*)q_latent, (const T*)up_keys, \
         norm_weight, eps, cos_sin, pairs, (T*)keys, (T*)values, table, table_stride, token_row, positions, page_size, (T*)out_q, heads, dim, \
-        rot_dim, rank, row_width, write_cache, n_tokens)
+        rot_dim, rank, row_width, write_cache, n_tokens, halves)
     if (code) LSA_LAUNCH(bf16_t); else LSA_LAUNCH(float);
 #undef LSA_LAUNCH
     LSA_LAUNCH_CHECK();

@@ -1,6 +1,7 @@
 // Kernels of the mixers that carry a state of fixed size from token to token: the mix of a token's row with the row
-// before it, the linear recurrence S_t = diag(d_t) S_(t-1) + k_t v_t^T with its read-out, the matrix memory with
-// exponential gates and a normaliser, and the per-head norm and gate behind them.  Decays, their exponentials and logarithms, the state, the sums and the norm are float32; projections
+// before it, the linear recurrence S_t = diag(d_t) S_(t-1) + k_t v_t^T with its read-out, the recurrences with one decay
+// per head (the matrix memory with exponential gates and a normaliser; the plain S_t = a_t S_(t-1) + b_t k_t v_t^T), and the
+// per-head norm and gate behind them.  Decays, their exponentials and logarithms, the state, the sums and the norm are float32; projections
 // arrive in the activations' type and are widened where they are read; a result for a 16-bit consumer is rounded once.
 #include "common.hpp"
 
@@ -190,7 +191,7 @@ __global__ __launch_bounds__(512) void linear_recurrence_kernel(const T* __restr
 }
 
 // grid (tokens, heads), one wavefront: out = x' / rms(x') * w * act(gate) over a head's value_dim numbers; x float32,
-// w = weight[head * weight_stride + j] (weight_stride 0: one weight shared by the heads), gate and out of type T;
+// w = weight[head * weight_stride + j] (weight_stride 0: one weight shared by the heads; no weight: 1), gate and out of type T;
 // act: gate * sigmoid(gate) (gate_kind 0) or sigmoid(gate) (1).  x' = x, or, with below [tokens][heads][2]:
 // x / (max(|below[0]|, below[1]) + floor), the read-out of a matrix memory under its normaliser.
 template <typename T>
@@ -212,13 +213,13 @@ __global__ __launch_bounds__(64) void heads_norm_gate_kernel(const float* __rest
     }
     const float inv = rsqrtf(wave_sum(sq) / (float)value_dim + eps);
     const T* g = gate + (size_t)t * gate_stride + (size_t)head * value_dim;
-    const float* w = weight + (size_t)head * weight_stride;
+    const float* w = weight ? weight + (size_t)head * weight_stride : nullptr;
     T* o = out + ((size_t)t * heads + head) * value_dim;
     for (int j = lane; j < value_dim; j += 64) {
         const float gv = (float)g[j];
         const float sigmoid = 1.f / (1.f + expf(-gv));
         const float xv = below ? row[j] / under : row[j];
-        o[j] = (T)(xv * inv * w[j] * (gate_kind ? sigmoid : gv * sigmoid));
+        o[j] = (T)(xv * inv * (w ? w[j] : 1.f) * (gate_kind ? sigmoid : gv * sigmoid));
     }
 }
 
@@ -333,7 +334,23 @@ __global__ __launch_bounds__(64 * GATES_WAVES) void memory_gates_kernel(const fl
     if (tid == 0) *kept = m;
 }
 
-// One token of one wavefront's DK channels of a matrix memory: S = keep S + k value (value: the token's value column times its
+// ---- recurrences with one decay per head: S_t = keep_t S_(t-1) + take_t k_t v_t^T, o_t = S_t^T q_t -------------------------
+// Where a token's two numbers of a head come from: pairs (keep, take) that another kernel has made (the matrix memory's
+// gates), or the logarithm of keep, per token and head or (log_stride 0) per head, with take per token and head or 1.
+struct DecayWeights {
+    const float* coef;                   // [T][heads][2], or nullptr: the two below
+    const float* log_keep;               // [T][heads] (log_stride = heads) or [heads] (log_stride = 0)
+    long log_stride;
+    const float* take;                   // [T][heads], or nullptr: 1
+    __device__ __forceinline__ float keep_of(size_t token, int head, int heads) const {
+        return coef ? coef[(token * heads + head) * 2] : expf(log_keep[token * log_stride + head]);
+    }
+    __device__ __forceinline__ float take_of(size_t token, int head, int heads) const {
+        return coef ? coef[(token * heads + head) * 2 + 1] : (take ? take[token * heads + head] : 1.f);
+    }
+};
+
+// One token of one wavefront's DK channels of such a recurrence: S = keep S + k value (value: the token's value column times its
 // take), and the channels' part of the read-out S^T q; the channels come from LDS as in recurrence_token.
 template <int DK>
 __device__ __forceinline__ float memory_token(float (&S)[DK], const float* q_row, const float* k_row, float keep, float value) {
@@ -356,17 +373,17 @@ __device__ __forceinline__ float memory_token(float (&S)[DK], const float* q_row
 
 // The memory itself, laid out as linear_recurrence_kernel: grid (rows, heads, blocks of 64 columns), lane = column,
 // wavefront w owns key channels [w * DK, (w + 1) * DK) and keeps its piece of the state in registers over the row's tokens.
-// The columns are the head's value_dim value columns and, behind them, one more whose "value" is 1: its piece of the state
-// is the normaliser n, which obeys the same recurrence with k in place of k v^T, and its read-out is n . q.  So
+// Groups of `group` heads share a query and key head.  The columns are the head's value_dim value columns and, with `ones`
+// (the matrix memory), behind them one more whose "value" is 1: its piece of the state is the normaliser n, which obeys the same recurrence with k in place of k v^T, and its read-out is n . q.  So
 // out [T][heads * value_dim] gets the numerators S^T q and below [T][heads][2] (first number) gets n . q; the division is
 // left to the kernel that normalises the heads.  state[slot]: the matrices [heads][dim][value_dim], then the normalisers
 // [heads][dim].  Every sum is formed in the same order however the sequence was cut into steps.
-template <typename T, int DK>
+template <typename T, typename V, int DK>
 __global__ __launch_bounds__(512) void matrix_memory_kernel(const T* __restrict__ q, long q_stride, const T* __restrict__ k, long k_stride,
-                                         const T* __restrict__ v, long v_stride, const float* __restrict__ coef, float q_scale,
+                                         const V* __restrict__ v, long v_stride, DecayWeights weights, float q_scale,
                                          float* state, long state_stride, const int* __restrict__ slots,
                                          const int* __restrict__ row_start, const int* __restrict__ row_len, const int* __restrict__ row_ctx,
-                                         float* __restrict__ out, float* __restrict__ below, int heads, int dim, int value_dim) {
+                                         float* __restrict__ out, float* __restrict__ below, int heads, int dim, int value_dim, int group, int ones) {
     extern __shared__ __align__(16) float lds[];
     const int row = blockIdx.x, head = blockIdx.y, column0 = blockIdx.z * 64;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, waves = blockDim.x >> 6;
@@ -380,7 +397,7 @@ __global__ __launch_bounds__(512) void matrix_memory_kernel(const T* __restrict_
     float* s_keep = s_v + CHUNK * 64;                    // [CHUNK]
     float* s_o = s_keep + CHUNK;                         // [waves][CHUNK][64]
     const int column = column0 + lane;
-    const bool is_value = column < value_dim, is_normaliser = column == value_dim;
+    const bool is_value = column < value_dim, is_normaliser = ones && column == value_dim;
     const int channel0 = wave * DK;
     float* slot = state + (size_t)slots[row] * state_stride;
     // a channel's number of this column: in the matrix, or in the normaliser behind the matrices
@@ -393,7 +410,7 @@ __global__ __launch_bounds__(512) void matrix_memory_kernel(const T* __restrict_
         const bool ok = (is_value || is_normaliser) && channel0 + i < dim;
         S[i] = (ok && first_position > 0) ? mine[(size_t)i * channel_stride] : 0.f;
     }
-    const size_t key_column = (size_t)head * dim;
+    const size_t key_column = (size_t)(head / group) * dim;
     for (int t0 = 0; t0 < count; t0 += CHUNK) {
         const int n = min(CHUNK, count - t0);
         __syncthreads();                                 // the chunk before has been read out of LDS
@@ -413,11 +430,11 @@ __global__ __launch_bounds__(512) void matrix_memory_kernel(const T* __restrict_
         for (int i = threadIdx.x; i < n * 64; i += blockDim.x) {
             const int t = i >> 6, c = column0 + (i & 63);
             const size_t token = (size_t)(start + t0 + t);
-            const float take = coef[(token * heads + head) * 2 + 1];
+            const float take = weights.take_of(token, head, heads);
             const float value = c < value_dim ? (float)v[token * v_stride + (size_t)head * value_dim + c] : (c == value_dim ? 1.f : 0.f);
             s_v[i] = take * value;
         }
-        if (threadIdx.x < n) s_keep[threadIdx.x] = coef[((size_t)(start + t0 + threadIdx.x) * heads + head) * 2];
+        if (threadIdx.x < n) s_keep[threadIdx.x] = weights.keep_of((size_t)(start + t0 + threadIdx.x), head, heads);
 #pragma unroll
         for (int j = 0; j < PER; ++j) {
             const int i = threadIdx.x + j * blockDim.x;
@@ -441,7 +458,7 @@ __global__ __launch_bounds__(512) void matrix_memory_kernel(const T* __restrict_
         __syncthreads();
         for (int i = threadIdx.x; i < n * 64; i += blockDim.x) {
             const int t = i >> 6, c = column0 + (i & 63);
-            if (c > value_dim) continue;
+            if (c >= value_dim + ones) continue;
             float total = 0.f;
             for (int w = 0; w < waves; ++w) total += s_o[(w * CHUNK + t) * 64 + (i & 63)];
             const size_t token = (size_t)(start + t0 + t);
@@ -454,14 +471,14 @@ __global__ __launch_bounds__(512) void matrix_memory_kernel(const T* __restrict_
         if ((is_value || is_normaliser) && channel0 + i < dim) mine[(size_t)i * channel_stride] = S[i];
 }
 
-// ---- the matrix memory in chunks -------------------------------------------------------------------------------------
+// ---- the same recurrences in chunks -------------------------------------------------------------------------------------
 // A row's tokens of a step in chunks of 64, counted from the row's first token of the step.  With L_t the sum of log keep
 // from the chunk's first token to t, the state behind token t is e^(L_t) S_0 + sum_(j <= t) e^(L_t - L_j) take_j k_j v_j^T
 // (S_0 the state in front of the chunk), and every weight is at most 1.  So (1) every chunk's own sum
 // U = sum_j e^(L_last - L_j) take_j k_j v_j^T is a matrix product, all chunks at once; (2) a walk over a row's chunks,
 // S <- e^(L_last) S + U, leaves the state in front of every chunk where U stood, and the row's last state in its slot; (3) a
 // chunk's read-outs are two products, (scores q_t . k_j times their weights) x values and (e^(L_t) q_t) x S_0, again all
-// chunks at once.  One more column behind the values, whose "value" is 1, carries the normaliser as in the scan.  All
+// chunks at once.  With `ones`, one more column behind the values, whose "value" is 1, carries the normaliser as in the scan.  All
 // operands are float32 in LDS and the products run on v_mfma_f32_16x16x4_f32; a workgroup of four wavefronts forms 64 x 64
 // results, a wavefront 32 x 32 of them.  An item is a (row, chunk): the grid has as many as the step could have at most,
 // and a workgroup finds its row by walking the rows' lengths.
@@ -508,6 +525,24 @@ __device__ __forceinline__ void memory_product(mc_f4 (&acc)[2][2], const float* 
     }
 }
 
+// L_t and take_t of a chunk's token `tid` (the first wavefront's lanes; lanes behind the chunk's n tokens: the last L, take 0):
+// from `run` and the pairs of coefficients where another kernel has summed the logarithms up, or summed here, in 64-bit.
+__device__ __forceinline__ void memory_chunk_weights(const DecayWeights& weights, const double* __restrict__ run, size_t token0, int n, int head,
+                                                     int heads, int lane, double& total, float& take) {
+    const size_t token = token0 + min(lane, n - 1);
+    take = lane < n ? weights.take_of(token, head, heads) : 0.f;
+    if (run != nullptr) {
+        total = run[token * heads + head];
+        return;
+    }
+    total = lane < n ? (double)weights.log_keep[token * weights.log_stride + head] : 0.0;
+#pragma unroll
+    for (int step = 1; step < 64; step <<= 1) {
+        const double other = __shfl_up(total, step, 64);
+        if (lane >= step) total += other;
+    }
+}
+
 // A chunk's values of 64 columns from column0 on, [token][column] in LDS: zeros behind the chunk's last token and behind the
 // column of ones that stands behind the values.  All of a thread's loads are issued before it stores.
 template <typename T>
@@ -528,12 +563,14 @@ __device__ __forceinline__ void memory_stage_values(float* s_v, const T* __restr
 }
 
 // (1) sums[item][head][channel][column] = sum_j e^(L_last - L_j) take_j k_j[channel] value_j[column]; grid (items, heads,
-// blocks of 64 columns of value_dim + 1), 256 threads.  A = the weighted keys, read as [channel][token]; B = the values.
-template <typename T>
-__global__ __launch_bounds__(256) void memory_chunk_sums_kernel(const T* __restrict__ k, long k_stride, const T* __restrict__ v, long v_stride,
-                                                                const float* __restrict__ coef, const double* __restrict__ run,
+// blocks of 64 columns of value_dim + ones), 256 threads.  A = the weighted keys, read as [channel][token]; B = the values.
+// totals (or nullptr) [item][head] = e^(L_last), for the walk.
+template <typename T, typename V>
+__global__ __launch_bounds__(256) void memory_chunk_sums_kernel(const T* __restrict__ k, long k_stride, const V* __restrict__ v, long v_stride,
+                                                                DecayWeights weights, const double* __restrict__ run,
                                                                 const int* __restrict__ row_start, const int* __restrict__ row_len, int rows,
-                                                                float* __restrict__ sums, int heads, int dim, int value_dim) {
+                                                                float* __restrict__ sums, float* __restrict__ totals, int heads, int dim,
+                                                                int value_dim, int group, int ones) {
     __shared__ float s_k[MC * MC_A];                     // [channel][token]
     __shared__ float s_v[MC * MC_B];                     // [token][column]
     __shared__ float s_w[MC];
@@ -542,14 +579,15 @@ __global__ __launch_bounds__(256) void memory_chunk_sums_kernel(const T* __restr
     const int head = blockIdx.y, column0 = blockIdx.z * 64, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int n = min(MC, row_len[row] - chunk * MC);
     const size_t token0 = (size_t)row_start[row] + (size_t)chunk * MC;
-    const int ld = value_dim + 1;
+    const int ld = value_dim + ones;
+    const size_t key_column = (size_t)(head / group) * dim;
     if (tid < MC) {
-        float w = 0.f;
-        if (tid < n) {
-            const double last = run[(token0 + n - 1) * heads + head];
-            w = expf((float)(last - run[(token0 + tid) * heads + head])) * coef[((token0 + tid) * heads + head) * 2 + 1];
-        }
-        s_w[tid] = w;
+        double total;
+        float take;
+        memory_chunk_weights(weights, run, token0, n, head, heads, tid, total, take);
+        const double last = __shfl(total, n - 1, 64);
+        s_w[tid] = expf((float)(last - total)) * take;
+        if (totals != nullptr && tid == 0 && blockIdx.z == 0) totals[(size_t)blockIdx.x * heads + head] = expf((float)last);
     }
     memory_stage_values(s_v, v, v_stride, token0, n, head, value_dim, column0, tid);
     const int mt = wave >> 1, nt = wave & 1;
@@ -559,7 +597,7 @@ __global__ __launch_bounds__(256) void memory_chunk_sums_kernel(const T* __restr
 #pragma unroll
         for (int j = 0; j < 16; ++j) {
             const int t = min(4 * j + (tid >> 6), n - 1), c = min(slab + (tid & 63), dim - 1);    // (neighbouring threads read neighbouring channels of one token)
-            keys[j] = k[(token0 + t) * k_stride + (size_t)head * dim + c];
+            keys[j] = k[(token0 + t) * k_stride + key_column + c];
         }
         __syncthreads();                                 // s_w is there; the slab before has been read
 #pragma unroll
@@ -568,7 +606,7 @@ __global__ __launch_bounds__(256) void memory_chunk_sums_kernel(const T* __restr
             s_k[c * MC_A + t] = (t < n && slab + c < dim) ? (float)keys[j] * s_w[t] : 0.f;
         }
         __syncthreads();
-        if (slab + mt * 32 >= dim || column0 + nt * 32 > value_dim) continue;
+        if (slab + mt * 32 >= dim || column0 + nt * 32 >= ld) continue;
         mc_f4 acc[2][2] = {};
         memory_product(acc, s_k + mt * 32 * MC_A, s_v + nt * 32, MC_B, 1, inner, lane);
         float* base = sums + (((size_t)blockIdx.x * heads + head) * dim) * ld;
@@ -579,21 +617,21 @@ __global__ __launch_bounds__(256) void memory_chunk_sums_kernel(const T* __restr
 #pragma unroll
                 for (int e = 0; e < 4; ++e) {
                     const int channel = slab + mt * 32 + 16 * mi + 4 * (lane >> 4) + e, column = column0 + nt * 32 + 16 * ni + (lane & 15);
-                    if (channel < dim && column <= value_dim) base[(size_t)channel * ld + column] = acc[mi][ni][e];
+                    if (channel < dim && column < ld) base[(size_t)channel * ld + column] = acc[mi][ni][e];
                 }
     }
 }
 
-// (2) grid (rows, heads, blocks of 256 numbers of a head's dim x (value_dim + 1)); a thread walks one number of the state
+// (2) grid (rows, heads, blocks of 256 numbers of a head's dim x (value_dim + ones)); a thread walks one number of the state
 // through the row's chunks.  The next chunk's sum is loaded before this chunk's place is overwritten.
-__global__ __launch_bounds__(256) void memory_chunk_carry_kernel(float* __restrict__ sums, const double* __restrict__ run, float* state, long state_stride,
+__global__ __launch_bounds__(256) void memory_chunk_carry_kernel(float* __restrict__ sums, const double* __restrict__ run, const float* __restrict__ totals, float* state, long state_stride,
                                                                  const int* __restrict__ slots, const int* __restrict__ row_start,
                                                                  const int* __restrict__ row_len, const int* __restrict__ row_ctx,
-                                                                 int heads, int dim, int value_dim) {
+                                                                 int heads, int dim, int value_dim, int ones) {
     const int row = blockIdx.x, head = blockIdx.y;
     const int count = row_len[row];
     if (count <= 0) return;
-    const int ld = value_dim + 1;
+    const int ld = value_dim + ones;
     const long e = (long)blockIdx.z * 256 + threadIdx.x;
     if (e >= (long)dim * ld) return;
     const int channel = (int)(e / ld), column = (int)(e - (long)channel * ld);
@@ -610,7 +648,7 @@ __global__ __launch_bounds__(256) void memory_chunk_carry_kernel(float* __restri
     for (int c = 0; c < chunks; ++c) {
         const float next = c + 1 < chunks ? place[step] : 0.f;
         const size_t last = (size_t)start + min(count, (c + 1) * MC) - 1;
-        const float keep = expf((float)run[last * heads + head]);
+        const float keep = totals ? totals[(size_t)(base + c) * heads + head] : expf((float)run[last * heads + head]);
         *place = S;
         S = __builtin_fmaf(keep, S, sum);
         sum = next;
@@ -620,14 +658,15 @@ __global__ __launch_bounds__(256) void memory_chunk_carry_kernel(float* __restri
 }
 
 // (3) out[t][head][column] = sum_(j <= t) (q_t . k_j) e^(L_t - L_j) take_j value_j[column] + e^(L_t) sum_channel q_t[channel] S_0[channel][column],
-// q scaled; the column behind the values goes to below[t][head][0].  grid and workgroup as in (1).
-template <typename T>
+// q scaled; with `ones` the column behind the values goes to below[t][head][0].  grid and workgroup as in (1).
+template <typename T, typename V>
 __global__ __launch_bounds__(256) void memory_chunk_read_kernel(const T* __restrict__ q, long q_stride, const T* __restrict__ k, long k_stride,
-                                                                const T* __restrict__ v, long v_stride, const float* __restrict__ coef,
+                                                                const V* __restrict__ v, long v_stride, DecayWeights weights,
                                                                 const double* __restrict__ run, float q_scale,
                                                                 const int* __restrict__ row_start, const int* __restrict__ row_len,
                                                                 const int* __restrict__ row_ctx, int rows, const float* __restrict__ sums,
-                                                                float* __restrict__ out, float* __restrict__ below, int heads, int dim, int value_dim) {
+                                                                float* __restrict__ out, float* __restrict__ below, int heads, int dim, int value_dim,
+                                                                int group, int ones) {
     __shared__ float s_q[MC * MC_A];                     // [token][channel]
     __shared__ float s_k[MC * MC_A];                     // [token][channel]; then the weighted scores [token t][token j]
     __shared__ float s_v[MC * MC_B];                     // [token or channel][column]
@@ -639,12 +678,16 @@ __global__ __launch_bounds__(256) void memory_chunk_read_kernel(const T* __restr
     const int count = row_len[row];
     const int n = min(MC, count - chunk * MC);
     const size_t token0 = (size_t)row_start[row] + (size_t)chunk * MC;
-    const int ld = value_dim + 1;
+    const int ld = value_dim + ones;
+    const size_t key_column = (size_t)(head / group) * dim;
     const bool from_zero = chunk == 0 && row_ctx[row] - count == 0;      // nothing stands in front of the sequence's first chunk
     if (tid < MC) {
-        s_run[tid] = tid < n ? run[(token0 + tid) * heads + head] : 0.0;
-        s_take[tid] = tid < n ? coef[((token0 + tid) * heads + head) * 2 + 1] : 0.f;
-        s_decay[tid] = expf((float)s_run[tid]);
+        double total;
+        float take;
+        memory_chunk_weights(weights, run, token0, n, head, heads, tid, total, take);
+        s_run[tid] = total;
+        s_take[tid] = take;
+        s_decay[tid] = expf((float)total);
     }
     const int mt = wave >> 1, nt = wave & 1;
     // the scores of the wavefront's 32 tokens t against 32 tokens j (nothing to do where every j lies behind every t)
@@ -654,8 +697,8 @@ __global__ __launch_bounds__(256) void memory_chunk_read_kernel(const T* __restr
 #pragma unroll
         for (int j = 0; j < 16; ++j) {
             const int t = min(4 * j + (tid >> 6), n - 1), c = min(slab + (tid & 63), dim - 1);
-            queries[j] = q[(token0 + t) * q_stride + (size_t)head * dim + c];
-            keys[j] = k[(token0 + t) * k_stride + (size_t)head * dim + c];
+            queries[j] = q[(token0 + t) * q_stride + key_column + c];
+            keys[j] = k[(token0 + t) * k_stride + key_column + c];
         }
         __syncthreads();
 #pragma unroll
@@ -682,7 +725,7 @@ __global__ __launch_bounds__(256) void memory_chunk_read_kernel(const T* __restr
             }
     memory_stage_values(s_v, v, v_stride, token0, n, head, value_dim, column0, tid);
     __syncthreads();
-    const bool wanted = column0 + nt * 32 <= value_dim;  // (uniform in a wavefront)
+    const bool wanted = column0 + nt * 32 < ld;  // (uniform in a wavefront)
     mc_f4 acc[2][2] = {};
     if (wanted) memory_product(acc, s_k + mt * 32 * MC_A, s_v + nt * 32, MC_B, 1, (mt + 1) * 32, lane);
     if (!from_zero) {
@@ -693,8 +736,8 @@ __global__ __launch_bounds__(256) void memory_chunk_read_kernel(const T* __restr
 #pragma unroll
             for (int j = 0; j < 16; ++j) {
                 const int t = 4 * j + (tid >> 6), c = tid & 63;          // queries [token][channel] times what the chunk's state has kept
-                queries[j] = q[(token0 + min(t, n - 1)) * q_stride + (size_t)head * dim + min(slab + c, dim - 1)];
-                const int channel = min(slab + t, dim - 1), column = min(column0 + c, value_dim);      // the state's slab [channel][column]
+                queries[j] = q[(token0 + min(t, n - 1)) * q_stride + key_column + min(slab + c, dim - 1)];
+                const int channel = min(slab + t, dim - 1), column = min(column0 + c, ld - 1);      // the state's slab [channel][column]
                 kept[j] = before[(size_t)channel * ld + column];
             }
             __syncthreads();
@@ -702,7 +745,7 @@ __global__ __launch_bounds__(256) void memory_chunk_read_kernel(const T* __restr
             for (int j = 0; j < 16; ++j) {
                 const int t = 4 * j + (tid >> 6), c = tid & 63;
                 s_q[t * MC_A + c] = (t < n && slab + c < dim) ? (float)queries[j] * q_scale * s_decay[t] : 0.f;
-                s_v[t * MC_B + c] = (slab + t < dim && column0 + c <= value_dim) ? kept[j] : 0.f;
+                s_v[t * MC_B + c] = (slab + t < dim && column0 + c < ld) ? kept[j] : 0.f;
             }
             __syncthreads();
             if (wanted) memory_product(acc, s_q + mt * 32 * MC_A, s_v + nt * 32, MC_B, 1, min(64, (dim - slab + 15) & ~15), lane);
@@ -716,7 +759,7 @@ __global__ __launch_bounds__(256) void memory_chunk_read_kernel(const T* __restr
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
                 const int t = mt * 32 + 16 * mi + 4 * (lane >> 4) + e, column = column0 + nt * 32 + 16 * ni + (lane & 15);
-                if (t >= n || column > value_dim) continue;
+                if (t >= n || column >= ld) continue;
                 if (column < value_dim) out[(token0 + t) * heads * value_dim + (size_t)head * value_dim + column] = acc[mi][ni][e];
                 else below[((token0 + t) * heads + head) * 2] = acc[mi][ni][e];
             }
@@ -786,13 +829,16 @@ LSA_EXPORT int lsa_recurrent_prepare() {
     LSA_ALLOW_ALL(bf16_t);
 #undef LSA_ALLOW_ALL
 #undef LSA_ALLOW
-#define LSA_ALLOW(T, DK) do { \
-        const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&matrix_memory_kernel<T, DK>), \
+#define LSA_ALLOW(T, V, DK) do { \
+        const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&matrix_memory_kernel<T, V, DK>), \
                                                  hipFuncAttributeMaxDynamicSharedMemorySize, MOST_LDS); \
         if (e != hipSuccess && first == hipSuccess) first = e; \
     } while (0)
-    LSA_ALLOW(float, 8); LSA_ALLOW(float, 16); LSA_ALLOW(float, 32); LSA_ALLOW(float, 64);
-    LSA_ALLOW(bf16_t, 8); LSA_ALLOW(bf16_t, 16); LSA_ALLOW(bf16_t, 32); LSA_ALLOW(bf16_t, 64);
+#define LSA_ALLOW_ALL(T, V) do { LSA_ALLOW(T, V, 8); LSA_ALLOW(T, V, 16); LSA_ALLOW(T, V, 32); LSA_ALLOW(T, V, 64); } while (0)
+    LSA_ALLOW_ALL(float, float);
+    LSA_ALLOW_ALL(bf16_t, bf16_t);
+    LSA_ALLOW_ALL(float, bf16_t);
+#undef LSA_ALLOW_ALL
 #undef LSA_ALLOW
     (void)hipGetLastError();
     return (int)first;
@@ -832,6 +878,40 @@ LSA_EXPORT int lsa_heads_norm_gate(int code, const float* x, const float* weight
     LSA_LAUNCH_CHECK();
 }
 
+// The recurrence itself, in either form; sums == nullptr: token by token.  In chunks, sums [items][heads][dim][value_dim + ones]
+// and, without `run`, totals [items][heads] are the caller's scratch memory; items is no less than the number of chunks of 64
+// tokens that the rows have together.
+template <typename T, typename V>
+static int run_decayed(const T* q, long q_stride, const T* k, long k_stride, const V* v, long v_stride, DecayWeights weights, const double* run,
+                       float q_scale, float* state, long state_stride, const int* slots, const int* row_start, const int* row_len,
+                       const int* row_ctx, float* out, float* below, int rows, int heads, int group, int dim, int value_dim, int ones,
+                       float* sums, float* totals, int items, hipStream_t stream) {
+    const int columns = value_dim + ones;
+    if (sums != nullptr) {
+        if (items <= 0 || (run == nullptr && totals == nullptr)) return -1;
+        const dim3 chunk_grid(items, heads, (columns + 63) / 64);
+        const dim3 carry_grid(rows, heads, (unsigned)(((long)dim * columns + 255) / 256));
+        memory_chunk_sums_kernel<T, V><<<chunk_grid, 256, 0, stream>>>(k, k_stride, v, v_stride, weights, run, row_start, row_len, rows, sums, totals,
+                                                                       heads, dim, value_dim, group, ones);
+        memory_chunk_carry_kernel<<<carry_grid, 256, 0, stream>>>(sums, run, totals, state, state_stride, slots, row_start, row_len, row_ctx, heads,
+                                                                  dim, value_dim, ones);
+        memory_chunk_read_kernel<T, V><<<chunk_grid, 256, 0, stream>>>(q, q_stride, k, k_stride, v, v_stride, weights, run, q_scale, row_start, row_len,
+                                                                       row_ctx, rows, sums, out, below, heads, dim, value_dim, group, ones);
+        LSA_LAUNCH_CHECK();
+    }
+    int dk, waves;
+    recurrence_lds(dim, dk, waves);
+    const size_t lds = sizeof(float) * ((size_t)2 * CHUNK * waves * dk + (size_t)CHUNK * 64 + CHUNK + (size_t)waves * CHUNK * 64);
+    if (lds > (size_t)MOST_LDS) return -1;
+    dim3 grid(rows, heads, (columns + 63) / 64);
+#define LSA_LAUNCH(DK) \
+        matrix_memory_kernel<T, V, DK><<<grid, waves * 64, lds, stream>>>(q, q_stride, k, k_stride, v, v_stride, weights, q_scale, state, state_stride, \
+            slots, row_start, row_len, row_ctx, out, below, heads, dim, value_dim, group, ones)
+    if (dk == 8) LSA_LAUNCH(8); else if (dk == 16) LSA_LAUNCH(16); else if (dk == 32) LSA_LAUNCH(32); else LSA_LAUNCH(64);
+#undef LSA_LAUNCH
+    LSA_LAUNCH_CHECK();
+}
+
 // state[slot]: the matrices [heads][dim][value_dim], the normalisers [heads][dim], the maxima [heads].
 LSA_EXPORT int lsa_matrix_memory(int code, const void* q, long q_stride, const void* k, long k_stride, const void* v, long v_stride,
                                  const float* gates, float cap, float q_scale, float* state, long state_stride, const int* slots,
@@ -839,40 +919,33 @@ LSA_EXPORT int lsa_matrix_memory(int code, const void* q, long q_stride, const v
                                  int rows, int heads, int dim, int value_dim, double* run, float* sums, int items, hipStream_t stream) {
     if (rows <= 0) return 0;
     if (dim < 1 || dim > MOST_DIM || value_dim < 1 || heads < 1 || !(cap > 0.f) || state == nullptr || coef == nullptr || below == nullptr) return -1;
-    if (state_stride < (long)heads * dim * value_dim + (long)heads * dim + heads) return -1;
-    int dk, waves;
-    recurrence_lds(dim, dk, waves);
-    const size_t lds = sizeof(float) * ((size_t)2 * CHUNK * waves * dk + (size_t)CHUNK * 64 + CHUNK + (size_t)waves * CHUNK * 64);
-    if (lds > (size_t)MOST_LDS) return -1;
+    if (state_stride < (long)heads * dim * value_dim + (long)heads * dim + heads || (run == nullptr) != (sums == nullptr)) return -1;
     memory_gates_kernel<<<dim3(rows, heads), 64 * GATES_WAVES, 0, stream>>>(gates, cap, state, state_stride, (long)heads * dim * value_dim + (long)heads * dim,
                                                               slots, row_start, row_len, row_ctx, coef, below, heads, run);
-    if (run != nullptr) {
-        // in chunks: run [T][heads] and sums [items][heads][dim][value_dim + 1] are the caller's scratch memory; items is no
-        // less than the number of chunks of 64 tokens that the rows have together
-        if (sums == nullptr || items <= 0) return -1;
-        const dim3 chunk_grid(items, heads, (value_dim + 1 + 63) / 64);
-        const dim3 carry_grid(rows, heads, (unsigned)(((long)dim * (value_dim + 1) + 255) / 256));
-#define LSA_CHUNKED(T) do { \
-            memory_chunk_sums_kernel<T><<<chunk_grid, 256, 0, stream>>>((const T*)k, k_stride, (const T*)v, v_stride, coef, run, row_start, row_len, rows, \
-                                                                        sums, heads, dim, value_dim); \
-            memory_chunk_carry_kernel<<<carry_grid, 256, 0, stream>>>(sums, run, state, state_stride, slots, row_start, row_len, row_ctx, heads, dim, value_dim); \
-            memory_chunk_read_kernel<T><<<chunk_grid, 256, 0, stream>>>((const T*)q, q_stride, (const T*)k, k_stride, (const T*)v, v_stride, coef, run, q_scale, \
-                                                                        row_start, row_len, row_ctx, rows, sums, out, below, heads, dim, value_dim); \
-        } while (0)
-        if (code) LSA_CHUNKED(bf16_t); else LSA_CHUNKED(float);
-#undef LSA_CHUNKED
-        LSA_LAUNCH_CHECK();
-    }
-    dim3 grid(rows, heads, (value_dim + 1 + 63) / 64);
-#define LSA_LAUNCH(T, DK) \
-        matrix_memory_kernel<T, DK><<<grid, waves * 64, lds, stream>>>((const T*)q, q_stride, (const T*)k, k_stride, (const T*)v, v_stride, \
-            coef, q_scale, state, state_stride, slots, row_start, row_len, row_ctx, out, below, heads, dim, value_dim)
-#define LSA_BY_DK(T) do { if (dk == 8) LSA_LAUNCH(T, 8); else if (dk == 16) LSA_LAUNCH(T, 16); else if (dk == 32) LSA_LAUNCH(T, 32); \
-                          else LSA_LAUNCH(T, 64); } while (0)
-    if (code) LSA_BY_DK(bf16_t); else LSA_BY_DK(float);
-#undef LSA_BY_DK
-#undef LSA_LAUNCH
-    LSA_LAUNCH_CHECK();
+    const DecayWeights weights{coef, nullptr, 0, nullptr};
+#define LSA_RUN(T) run_decayed<T, T>((const T*)q, q_stride, (const T*)k, k_stride, (const T*)v, v_stride, weights, run, q_scale, state, state_stride, \
+                                     slots, row_start, row_len, row_ctx, out, below, rows, heads, 1, dim, value_dim, 1, sums, nullptr, items, stream)
+    return code ? LSA_RUN(bf16_t) : LSA_RUN(float);
+#undef LSA_RUN
+}
+
+// S_t = exp(log_keep) S_(t-1) + take k_t v_t^T, out_t = S_t^T (q_t q_scale) per head; groups of `group` heads share a query and a
+// key head; queries and keys of one type, values of the same or, behind float32 queries and keys, bfloat16.
+// state[slot]: the matrices [heads][dim][value_dim].
+LSA_EXPORT int lsa_decayed_recurrence(int key_code, const void* q, long q_stride, const void* k, long k_stride, int value_code, const void* v,
+                                      long v_stride, const float* log_keep, long log_stride, const float* take, float q_scale, float* state,
+                                      long state_stride, const int* slots, const int* row_start, const int* row_len, const int* row_ctx, float* out,
+                                      int rows, int heads, int group, int dim, int value_dim, float* sums, float* totals, int items,
+                                      hipStream_t stream) {
+    if (rows <= 0) return 0;
+    if (dim < 1 || dim > MOST_DIM || value_dim < 1 || heads < 1 || group < 1 || heads % group || state == nullptr || log_keep == nullptr) return -1;
+    if ((log_stride != 0 && log_stride != heads) || (key_code && !value_code)) return -1;
+    const DecayWeights weights{nullptr, log_keep, log_stride, take};
+#define LSA_RUN(T, V) run_decayed<T, V>((const T*)q, q_stride, (const T*)k, k_stride, (const V*)v, v_stride, weights, nullptr, q_scale, state, state_stride, \
+                                        slots, row_start, row_len, row_ctx, out, nullptr, rows, heads, group, dim, value_dim, 0, sums, totals, items, stream)
+    if (key_code) return LSA_RUN(bf16_t, bf16_t);
+    return value_code ? LSA_RUN(float, bf16_t) : LSA_RUN(float, float);
+#undef LSA_RUN
 }
 
 LSA_EXPORT int lsa_tanh(int code, void* x, long n, hipStream_t stream) {

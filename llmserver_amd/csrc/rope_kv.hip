@@ -1,7 +1,7 @@
 // Per-head q/k RMSNorm, rotate-half rotation and the write of new keys and values into their
 // pages, for all tokens of the step (portions of prompts and decoded tokens alike).
 //
-// rotary_table: cos and sin of position * inv_freq for every token of the step, once per step
+// rotary_table: cos and sin of position * inv_freq, times a constant, for every token of the step, once per step
 //   (the angles depend on the token and the pair of dimensions only, not on the layer or head).
 // qk_norm_rope_kv_write: d / 16 lanes per (token, head), vector accesses throughout.  q heads are
 //   normalised, rotated and written back in place into the projection buffer; k heads are
@@ -16,13 +16,13 @@
 using namespace lsa;
 
 __global__ void rotary_table_kernel(const int* __restrict__ positions, const float* __restrict__ inv_freq,
-                                    float* __restrict__ cos_sin, int half, int n_tokens) {
+                                    float* __restrict__ cos_sin, int half, int n_tokens, float amplitude) {
     const int i = blockIdx.x * blockDim.x + threadIdx.x;
     if (i >= n_tokens * half) return;
     const int token = i / half, pair = i % half;
     const float angle = (float)positions[token] * inv_freq[pair];
-    cos_sin[(size_t)token * 2 * half + pair] = cosf(angle);
-    cos_sin[(size_t)token * 2 * half + half + pair] = sinf(angle);
+    cos_sin[(size_t)token * 2 * half + pair] = amplitude * cosf(angle);
+    cos_sin[(size_t)token * 2 * half + half + pair] = amplitude * sinf(angle);
 }
 
 // A (token, head) pair is handled by d / 16 neighbouring lanes: lane j of them owns dimensions
@@ -251,10 +251,10 @@ static int launch(void* qkv, void* keys, void* values, const int* table, int tab
     LSA_LAUNCH_CHECK();
 }
 
-LSA_EXPORT int lsa_rotary_table(const int* positions, const float* inv_freq, float* cos_sin, int half, int n_tokens, hipStream_t stream) {
+LSA_EXPORT int lsa_rotary_table(const int* positions, const float* inv_freq, float* cos_sin, int half, int n_tokens, float amplitude, hipStream_t stream) {
     const int total = n_tokens * half;
     if (total <= 0) return 0;
-    rotary_table_kernel<<<(total + 255) / 256, 256, 0, stream>>>(positions, inv_freq, cos_sin, half, n_tokens);
+    rotary_table_kernel<<<(total + 255) / 256, 256, 0, stream>>>(positions, inv_freq, cos_sin, half, n_tokens, amplitude);
     LSA_LAUNCH_CHECK();
 }
 

@@ -197,6 +197,52 @@ __global__ __launch_bounds__(256) void embedding_wide_kernel(const T* __restrict
     }
 }
 
+// One stream in front of a pass over a run of layers: x[t] += table[ids[t]] * scale (scale 0: nothing) + vector, where x lies,
+// and, where next_weight is given, normed = rmsnorm(x) * next_weight.  One workgroup a token; a thread issues the loads of its
+// first INJECT_COLS columns before it stores; longer rows are walked, and read again by the thread that wrote them.
+constexpr int INJECT_COLS = 8;
+template <typename T, typename R>
+__global__ __launch_bounds__(256) void stream_inject_kernel(float* __restrict__ x, const T* __restrict__ table, const int* __restrict__ ids,
+                                                            float scale, const float* __restrict__ vector, const float* __restrict__ next_weight,
+                                                            float eps, R* __restrict__ normed, int width, int vocab) {
+    __shared__ float scratch[16];
+    float* row = x + (size_t)blockIdx.x * width;
+    const int id = ids[blockIdx.x];
+    const float times = id >= 0 && id < vocab ? scale : 0.f;
+    const T* start = table + (size_t)(id >= 0 && id < vocab ? id : 0) * width;
+    const float* following = next_weight ? next_weight : vector;
+    float kept[INJECT_COLS], weights[INJECT_COLS];
+    float sq = 0.f;
+#pragma unroll
+    for (int k = 0; k < INJECT_COLS; ++k) {
+        const int i = min((int)threadIdx.x + k * 256, width - 1);
+        kept[k] = row[i] + times * (float)start[i] + vector[i];
+        weights[k] = following[i];
+    }
+#pragma unroll
+    for (int k = 0; k < INJECT_COLS; ++k) {
+        const int i = threadIdx.x + k * 256;
+        if (i < width) {
+            row[i] = kept[k];
+            sq += kept[k] * kept[k];
+        }
+    }
+    for (int i = threadIdx.x + INJECT_COLS * 256; i < width; i += 256) {
+        const float u = row[i] + times * (float)start[i] + vector[i];
+        row[i] = u;
+        sq += u * u;
+    }
+    if (!next_weight) return;
+    const float inv = rsqrtf(block_sum(sq, scratch) / (float)width + eps);
+    R* o = normed + (size_t)blockIdx.x * width;
+#pragma unroll
+    for (int k = 0; k < INJECT_COLS; ++k) {
+        const int i = threadIdx.x + k * 256;
+        if (i < width) o[i] = (R)(kept[k] * inv * weights[k]);
+    }
+    for (int i = threadIdx.x + INJECT_COLS * 256; i < width; i += 256) o[i] = (R)(row[i] * inv * next_weight[i]);
+}
+
 // ---- several residual streams x [S][T][W], float32 ------------------------------------------------------------------------
 constexpr int MOST_STREAMS = 8;
 constexpr int STREAM_CACHE = 8;           // elements of a row a thread keeps between the two passes (rows of up to 2,048 are read once; sixteen gained nothing at 4,096 and cost a prompt a little)
@@ -413,6 +459,20 @@ LSA_EXPORT int lsa_embedding_wide(int table_code, const void* table, const int* 
     const size_t copy_stride = (size_t)n * width;
     if (table_code) embedding_wide_kernel<bf16_t><<<n, 256, 0, stream>>>((const bf16_t*)table, ids, out, width, vocab, scale, copies, copy_stride);
     else embedding_wide_kernel<float><<<n, 256, 0, stream>>>((const float*)table, ids, out, width, vocab, scale, copies, copy_stride);
+    LSA_LAUNCH_CHECK();
+}
+
+LSA_EXPORT int lsa_stream_inject(float* x, int table_code, const void* table, const int* ids, float scale, const float* vector,
+                                 const float* next_weight, float eps, void* normed, int normed_code, int n, int width, int vocab,
+                                 hipStream_t stream) {
+    if (n <= 0) return 0;
+    if (next_weight != nullptr && normed == nullptr) return -1;
+#define LSA_LAUNCH(T, R) stream_inject_kernel<T, R><<<n, 256, 0, stream>>>(x, (const T*)table, ids, scale, vector, next_weight, eps, (R*)normed, width, vocab)
+    if (table_code && normed_code) LSA_LAUNCH(bf16_t, bf16_t);
+    else if (table_code) LSA_LAUNCH(bf16_t, float);
+    else if (normed_code) LSA_LAUNCH(float, bf16_t);
+    else LSA_LAUNCH(float, float);
+#undef LSA_LAUNCH
     LSA_LAUNCH_CHECK();
 }
 

@@ -52,7 +52,7 @@ def _flops(spec: ParamSpec, rows: int) -> float:
 
 def _weights(model) -> Dict[str, Iterable[ParamSpec]]:
     return {"embedding": model.embedding.param_specs().values(),
-            "blocks": [spec for block in model.blocks for spec in block.param_specs().values()],
+            "blocks": [spec for part in (*model.extras.values(), *model.blocks) for spec in part.param_specs().values()],
             "final_norm": model.final_norm.param_specs().values(), "head": model.head.param_specs().values()}
 
 

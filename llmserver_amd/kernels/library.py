@@ -17,7 +17,7 @@ _SIGNATURES = {
     "lsa_plain_read": [_P, _P, c_long, c_int, c_int, _P],
     "lsa_qk_norm_rope_kv_write": [c_int, _P, _P, _P, _P, c_int, _P, _P, _P, _P, c_float, _P, c_int, c_int, c_int, c_int,
                                   c_int, c_int, _P],
-    "lsa_rotary_table": [_P, _P, _P, c_int, c_int, _P],
+    "lsa_rotary_table": [_P, _P, _P, c_int, c_int, c_float, _P],
     "lsa_sample": [_P, _P, _P, _P, _P, c_int, c_int, _P],
     "lsa_sample_chunks": [c_int],
     "lsa_sample_static": [_P, _P, _P, _P, c_int, c_int, _P],
@@ -26,12 +26,18 @@ _SIGNATURES = {
     "lsa_paged_attention": [_P, c_long, _P, _P, _P, _P, c_int, _P, _P, _P, _P, _P, c_int, _P, c_int, c_int, _P, _P, _P, _P, c_int,
                             c_float, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, _P, _P, c_float, _P, c_int, c_int, c_int, _P, c_float, _P],
     "lsa_embedding_wide": [c_int, _P, _P, _P, c_int, c_int, c_int, c_float, c_int, _P],
+    "lsa_stream_inject": [_P, c_int, _P, _P, c_float, _P, _P, c_float, _P, c_int, c_int, c_int, c_int, _P],
     "lsa_most_streams": [],
     "lsa_streams_read": [_P, c_int, c_int, _P, _P, _P, c_float, _P, c_int, c_int, c_int, _P],
     "lsa_streams_update": [_P, c_int, c_int, _P, c_int, _P, _P, _P, _P, c_float, _P, c_int, c_int, _P],
     "lsa_activation": [c_int, _P, c_long, c_int, _P],
     "lsa_matrix_memory": [c_int, _P, c_long, _P, c_long, _P, c_long, _P, c_float, c_float, _P, c_long, _P, _P, _P, _P, _P, _P, _P,
                           c_int, c_int, c_int, c_int, _P, _P, c_int, _P],
+    "lsa_decayed_recurrence": [c_int, _P, c_long, _P, c_long, c_int, _P, c_long, _P, c_long, _P, c_float, _P, c_long, _P, _P, _P, _P, _P,
+                               c_int, c_int, c_int, c_int, c_int, _P, _P, c_int, _P],
+    "lsa_ssd_prepare": [c_int, _P, c_long, _P, c_int, _P, _P, c_long, _P, _P, _P, _P, _P, c_int, c_int, _P, c_long, _P, _P, _P, _P, c_int, c_int, _P],
+    "lsa_gated_group_norm": [c_int, _P, _P, c_long, _P, _P, c_long, _P, c_float, _P, c_int, c_int, c_int, c_int, _P],
+    "lsa_rotate_heads": [c_int, _P, c_long, _P, c_long, _P, c_int, c_float, _P, _P, c_int, c_int, c_int, _P],
     "lsa_norm_add_norm": [_P, _P, _P, c_int, c_float, c_float, _P, c_float, _P, _P, c_float, _P, c_int, c_int, c_int, _P],
     "lsa_qkv_prepare": [c_int, _P, c_long, _P, _P, _P, c_int, _P, _P, _P, _P, c_float, _P, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
                         _P, c_int, c_int, c_int, c_int, _P],
@@ -50,10 +56,10 @@ _SIGNATURES = {
     "lsa_short_conv_keep": [_P, _P, _P, _P, _P, _P, c_int, c_int, c_int, _P],
     "lsa_scaled_norm_add": [_P, _P, c_int, _P, _P, c_float, _P, _P, c_int, _P, c_long, c_int, _P, c_int, c_int, _P],
     "lsa_latent_prepare": [c_int, _P, c_long, _P, _P, _P, c_float, _P, c_int, _P, _P, _P, c_int, _P, _P, c_int, _P, c_int, c_int, c_int,
-                           c_int, c_int, c_int, c_int, _P],
+                           c_int, c_int, c_int, c_int, c_int, _P],
     "lsa_gate_heads": [c_int, _P, _P, _P, c_int, c_int, _P, c_long, c_int, _P, c_int, c_int, c_int, c_int, _P],
     "lsa_route_logits": [_P, _P, _P, c_int, c_int, c_int, _P],
-    "lsa_route_top": [_P, c_int, c_int, _P, _P, c_int, c_int, c_int, c_int, _P, _P],
+    "lsa_route_top": [_P, c_int, c_int, _P, _P, c_int, c_int, c_int, c_int, _P, _P, c_float, c_int, _P, _P],
     "lsa_gated_pair_update": [_P, _P, c_int, c_int, _P, c_int, _P, _P, c_int, _P, _P, c_float, _P, c_int, c_int, c_int, _P],
     "lsa_differential_heads": [c_int, _P, c_float, c_float, c_float, _P, c_int, c_int, c_int, c_int, c_int, _P],
     "lsa_delta_most_dim": [],
@@ -62,10 +68,10 @@ _SIGNATURES = {
                           _P, c_long, _P, c_long, c_int, _P, _P, _P, _P, c_int, _P],
     "lsa_delta_conv_keep": [c_int, _P, c_long, _P, c_long, _P, _P, _P, _P, c_int, c_int, c_int, _P],
     "lsa_delta_rule": [_P, _P, _P, c_int, _P, c_long, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, _P],
-    "lsa_experts_gate_up": [c_int, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_float, _P],
+    "lsa_experts_gate_up": [c_int, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_float, c_int, _P, _P, c_int, _P],
     "lsa_experts_tile_rows": [],
-    "lsa_experts_tiled": [_P, _P, _P, _P, _P, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int, c_float, _P],
-    "lsa_experts_down": [c_int, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, _P],
+    "lsa_experts_tiled": [_P, _P, _P, _P, _P, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, _P, _P, _P],
+    "lsa_experts_down": [c_int, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, _P, _P, _P, _P, _P, c_int, _P],
     "lsa_attention_workgroup_tiles": [],
     "lsa_attention_tile_page_multiple": [],
     "lsa_attention_tile_halves": [],

@@ -619,13 +619,14 @@ class HipOps(KernelNamespace):
         _check(bias, "bias", torch.float32, (width,))
         _launched(self._elementwise.lsa_add_bias(_code(y), _ptr(y), _ptr(bias), n, width, _stream()), "add_bias")
 
-    def rotary_table(self, positions, inv_freq):
-        """cos and sin of ``position * inv_freq`` for every token: float32 ``[T, 2 * len(inv_freq)]``, cos first."""
+    def rotary_table(self, positions, inv_freq, amplitude=1.0):
+        """cos and sin of ``position * inv_freq``, times ``amplitude``, for every token: float32 ``[T, 2 * len(inv_freq)]``, cos first."""
         n, half = positions.shape[0], inv_freq.shape[0]
         _check(positions, "positions", torch.int32)
         _check(inv_freq, "inv_freq", torch.float32)
         out = torch.empty((n, 2 * half), device=positions.device, dtype=torch.float32)
-        _launched(self._rope_kv.lsa_rotary_table(_ptr(positions), _ptr(inv_freq), _ptr(out), half, n, _stream()), "rotary_table")
+        _launched(self._rope_kv.lsa_rotary_table(_ptr(positions), _ptr(inv_freq), _ptr(out), half, n, float(amplitude), _stream()),
+                  "rotary_table")
         return out
 
     def qk_norm_rope_kv_write(self, qkv, keys, values, table, token_row, positions, q_weight, k_weight, eps, cos_sin,
@@ -821,6 +822,20 @@ class HipOps(KernelNamespace):
         _launched(self._part_library("stream").lsa_embedding_wide(_code(table), _ptr(table), _ptr(token_ids), _ptr(out), n, width,
                                                                   table.shape[0], float(scale), copies, _stream()), "embedding_wide")
 
+    def stream_inject(self, x, table, token_ids, scale, vector, next_weight=None, next_eps=0.0, normed=None):
+        n, width = x.shape
+        _check(x, "x", torch.float32)
+        _check(table, "table", None, (table.shape[0], width))
+        _check(token_ids, "token_ids", torch.int32, (n,))
+        _check(vector, "vector", torch.float32, (width,))
+        if next_weight is not None:
+            _check(next_weight, "next_weight", torch.float32, (width,))
+            _check(normed, "normed", None, (n, width))
+        _launched(self._part_library("stream").lsa_stream_inject(
+            _ptr(x), _code(table), _ptr(table), _ptr(token_ids), float(scale), _ptr(vector), _ptr(next_weight), float(next_eps),
+            _ptr(normed) if next_weight is not None else None, _code(normed) if next_weight is not None else 0, n, width, table.shape[0],
+            _stream()), "stream_inject")
+
     def _check_streams(self, streams):
         _check(streams, "streams", torch.float32)
         most = self._part_library("stream").lsa_most_streams()
@@ -952,7 +967,9 @@ class HipOps(KernelNamespace):
         return 0 < n_tokens <= self.LATENT_FEW_ROWS
 
     def latent_prepare(self, proj, q_latent, norm_weight, eps, cos_sin, keys, values, table, token_row, positions, page_size,
-                       out_q, n_heads, dim, rot_dim, rank, write_cache=True, up_keys=None):
+                       out_q, n_heads, dim, rot_dim, rank, write_cache=True, up_keys=None, pairing="neighbours"):
+        if pairing not in ("neighbours", "halves"):
+            raise ValueError(f"rotated dimensions pair up as neighbours or as halves, not {pairing!r}")
         n = proj.shape[0]
         _check(proj, "proj")
         if proj.shape[1] < n_heads * (dim + rot_dim) + rank + rot_dim:
@@ -980,7 +997,7 @@ class HipOps(KernelNamespace):
         _launched(self._part_library("latent").lsa_latent_prepare(
             _code(proj), _ptr(proj), proj.shape[1], _ptr(q_latent), _ptr(up_keys), _ptr(norm_weight), float(eps), _ptr(cos_sin), pairs,
             _ptr(keys), _ptr(values), _ptr(table), table.shape[1], _ptr(token_row), _ptr(positions), page_size, _ptr(out_q), n_heads, dim,
-            rot_dim, rank, row_width, 1 if write_cache else 0, n, _stream()), "latent_prepare")
+            rot_dim, rank, row_width, 1 if write_cache else 0, n, 1 if pairing == "halves" else 0, _stream()), "latent_prepare")
 
     def gate_heads(self, y, proj, gate_column, out, mixed=None, up_values=None, per_channel=False):
         _check(proj, "proj", out.dtype)
@@ -1006,34 +1023,44 @@ class HipOps(KernelNamespace):
                                                               proj.shape[1], int(gate_column), _ptr(out), heads, v, n, 1 if per_channel else 0,
                                                               _stream()), "gate_heads")
 
-    def route_experts(self, x, router, top, chosen, weights, scoring="softmax", groups=None, bias=None):
+    SCORINGS = ("softmax", "sigmoid", "softmax_all")       # (the kernel's codes)
+
+    def route_experts(self, x, router, top, chosen, weights, scoring="softmax", groups=None, bias=None, correction=None, weight_scale=1.0,
+                      gate_out=None):
         """The logits are a float32 product of the library (no reduced-precision mode), the choice and the weights a kernel
         (which also adds the bias)."""
         n, width = x.shape
-        experts = router.shape[0]
+        outputs = router.shape[0]
+        experts = outputs - (1 if gate_out is not None else 0)          # (the row behind the experts' is the gate's)
         _check(x, "x")
-        _check(router, "router", torch.float32, (experts, width))
+        _check(router, "router", torch.float32, (outputs, width))
         _check(chosen, "chosen", torch.int32, (n, top))
         _check(weights, "weights", torch.float32, (n, top))
         if bias is not None:
             _check(bias, "bias", torch.float32, (experts,))
+        if correction is not None:
+            _check(correction, "correction", torch.float32, (experts,))
+        if gate_out is not None:
+            _check(gate_out, "gate_out", torch.float32, (n,))
         if not 1 <= top <= experts or experts > 3072:
             raise ValueError(f"the router kernel chooses 1 to {min(experts, 3072)} of up to 3072 experts, asked for {top} of {experts}")
         wide = x if x.dtype == torch.float32 else x.float()
         if n <= self.LATENT_FEW_ROWS:          # few tokens: a kernel of a few microseconds instead of a library call
-            logits = torch.empty((n, experts), device=x.device, dtype=torch.float32)
-            _launched(self._part_library("experts").lsa_route_logits(_ptr(wide), _ptr(router), _ptr(logits), n, experts, width, _stream()),
+            logits = torch.empty((n, outputs), device=x.device, dtype=torch.float32)
+            _launched(self._part_library("experts").lsa_route_logits(_ptr(wide), _ptr(router), _ptr(logits), n, outputs, width, _stream()),
                       "route_logits")
         else:
             logits = torch.mm(wide, router.t())
-        if scoring not in ("softmax", "sigmoid") or (groups is not None and scoring != "sigmoid"):
-            raise ValueError(f"the router kernel scores by softmax or sigmoid (groups with sigmoid only), asked for {scoring!r}, groups {groups}")
+        if scoring not in self.SCORINGS or (groups is not None and scoring != "sigmoid"):
+            raise ValueError(f"the router kernel scores by {self.SCORINGS} (groups with sigmoid only), asked for {scoring!r}, groups {groups}")
+        if (correction is not None or weight_scale != 1.0) and scoring != "softmax_all":
+            raise ValueError("a correction of the choice and a scale of the weights come with the softmax over all experts")
         count, keep = groups if groups is not None else (1, 1)
         if count > 64 or experts % count or not 1 <= keep <= count or top > keep * (experts // count):
             raise ValueError(f"the router kernel takes up to 64 equal groups: {experts} experts in {count} groups, {keep} kept, {top} chosen")
         _launched(self._part_library("experts").lsa_route_top(_ptr(logits), experts, top, _ptr(chosen), _ptr(weights), n,
-                                                              1 if scoring == "sigmoid" else 0, int(count), int(keep), _ptr(bias), _stream()),
-                  "route_top")
+                                                              self.SCORINGS.index(scoring), int(count), int(keep), _ptr(bias), _ptr(correction),
+                                                              float(weight_scale), outputs, _ptr(gate_out), _stream()), "route_top")
 
     @staticmethod
     def _expert_limit(activation, limit) -> float:
@@ -1044,18 +1071,34 @@ class HipOps(KernelNamespace):
             raise ValueError(f"the experts' kernels compute silu, or the clamped form with a positive limit; asked for {activation!r}, {limit}")
         return float(limit)
 
-    def experts_gate_up(self, x, gate_up, chosen, hidden, activation="silu", limit=0.0):
+    def experts_gate_up(self, x, gate_up, chosen, hidden, activation="silu", limit=0.0, identity=0, shared=None):
         n, width = x.shape
         experts, top, inter = gate_up.shape[0], chosen.shape[1], hidden.shape[1]
         _check(x, "x")
         _check(gate_up, "gate_up", x.dtype, (experts, 2 * inter, width))
         _check(chosen, "chosen", torch.int32, (n, top))
         _check(hidden, "hidden", x.dtype, (n * top, inter))
+        shared_inter = 0
+        if shared is not None:
+            shared_inter = shared[1].shape[1]
+            _check(shared[0], "the shared expert's gate_up", x.dtype, (2 * shared_inter, width))
+            _check(shared[1], "the shared expert's hidden", x.dtype, (n, shared_inter))
         _launched(self._part_library("experts").lsa_experts_gate_up(_code(x), _ptr(x), _ptr(gate_up), _ptr(chosen), _ptr(hidden), n, top,
-                                                                    inter, width, experts, self._expert_limit(activation, limit), _stream()),
+                                                                    inter, width, experts, self._expert_limit(activation, limit), int(identity),
+                                                                    _ptr(shared[0]) if shared is not None else None,
+                                                                    _ptr(shared[1]) if shared is not None else None, shared_inter, _stream()),
                   "experts_gate_up")
 
-    def experts_down(self, hidden, down, chosen, weights, out):
+    @staticmethod
+    def _check_beside(like, n, width, x, shared_y, shared_gate):
+        if x is not None:
+            _check(x, "x", like.dtype, (n, width))
+        if shared_y is not None:
+            _check(shared_y, "shared_y", like.dtype, (n, width))
+        if shared_gate is not None:
+            _check(shared_gate, "shared_gate", torch.float32, (n,))
+
+    def experts_down(self, hidden, down, chosen, weights, out, x=None, shared=None, shared_y=None, shared_gate=None):
         n, width = out.shape
         experts, top, inter = down.shape[0], chosen.shape[1], hidden.shape[1]
         _check(hidden, "hidden", None, (n * top, inter))
@@ -1063,10 +1106,27 @@ class HipOps(KernelNamespace):
         _check(chosen, "chosen", torch.int32, (n, top))
         _check(weights, "weights", torch.float32, (n, top))
         _check(out, "out", torch.float32)
+        self._check_beside(hidden, n, width, x, shared_y, shared_gate)
+        if (shared_gate is None) != (shared is None and shared_y is None) or (shared is not None and shared_y is not None):
+            raise ValueError("a shared expert comes with its gate, and as its output or as its matrix and hidden rows")
+        shared_inter = 0
+        if shared is not None:
+            shared_inter = shared[1].shape[1]
+            _check(shared[0], "the shared expert's down", hidden.dtype, (width, shared_inter))
+            _check(shared[1], "the shared expert's hidden", hidden.dtype, (n, shared_inter))
         _launched(self._part_library("experts").lsa_experts_down(_code(hidden), _ptr(hidden), _ptr(down), _ptr(chosen), _ptr(weights),
-                                                                 _ptr(out), n, top, inter, width, experts, _stream()), "experts_down")
+                                                                 _ptr(out), n, top, inter, width, experts, _ptr(x), _ptr(shared_gate), _ptr(shared_y),
+                                                                 _ptr(shared[0]) if shared is not None else None,
+                                                                 _ptr(shared[1]) if shared is not None else None, shared_inter, _stream()),
+                  "experts_down")
 
-    def experts_sorted(self, x, gate_up, down, chosen, weights, out, activation="silu", limit=0.0) -> bool:
+    SHARED_INSIDE_ROWS = 4      # up to this many tokens the shared expert's products are made inside the routed experts' kernels
+
+    def shared_expert_inside(self, n_tokens: int) -> bool:
+        return 0 < n_tokens <= self.SHARED_INSIDE_ROWS
+
+    def experts_sorted(self, x, gate_up, down, chosen, weights, out, activation="silu", limit=0.0, identity=0, shared_y=None,
+                       shared_gate=None) -> bool:
         """Offered in bfloat16 for widths and expert sizes in steps of 32, and taken where the step has more (token,
         expert) pairs than there are experts: below that every pair streaming its own expert reads no more."""
         n, width = x.shape
@@ -1079,6 +1139,7 @@ class HipOps(KernelNamespace):
         _check(chosen, "chosen", torch.int32, (n, top))
         _check(weights, "weights", torch.float32, (n, top))
         _check(out, "out", torch.float32, (n, width))
+        self._check_beside(x, n, width, None, shared_y, shared_gate)
         lib = self._part_library("experts")
         tile = lib.lsa_experts_tile_rows()
         max_tiles = -(-n * top // tile) + experts
@@ -1087,7 +1148,8 @@ class HipOps(KernelNamespace):
         scratch = torch.empty((max_tiles * (tile + 1),), device=x.device, dtype=torch.int32)
         _launched(lib.lsa_experts_tiled(_ptr(x), _ptr(gate_up), _ptr(down), _ptr(chosen), _ptr(weights), _ptr(hidden), _ptr(y), _ptr(out),
                                         _ptr(scratch), scratch[max_tiles * tile:].data_ptr(), max_tiles, n, top, inter, width, experts,
-                                        self._expert_limit(activation, limit), _stream()), "experts_tiled")
+                                        self._expert_limit(activation, limit), int(identity), _ptr(shared_gate), _ptr(shared_y), _stream()),
+                  "experts_tiled")
         return True
 
     # -- general preparation of queries, keys and values; mixers with a recurrent state -----------------------------
@@ -1360,13 +1422,107 @@ class HipOps(KernelNamespace):
         if below is not None:
             _check(below, "below", torch.float32, (n, heads, 2))
         _check(x, "x", torch.float32, (n, heads * value_dim))
-        _check(weight, "weight", torch.float32, (heads * value_dim if weight_per_channel else value_dim,))
+        if weight is not None:
+            _check(weight, "weight", torch.float32, (heads * value_dim if weight_per_channel else value_dim,))
         _check(out, "out", None, (n, heads * value_dim))
         if not gate.is_cuda or gate.dtype != out.dtype or tuple(gate.shape) != (n, heads * value_dim) or (n > 1 and gate.stride(1) != 1):
             raise ValueError(f"gate must be a view [{n}, {heads * value_dim}] of {out.dtype} on the GPU with unit stride along a row")
         _launched(self._part_library("recurrent").lsa_heads_norm_gate(
             _code(out), _ptr(x), _ptr(weight), 1 if weight_per_channel else 0, float(eps), gate.data_ptr(), gate.stride(0), _ptr(out),
             n, heads, value_dim, self.GATE_ACTIVATIONS.index(gate_activation), _ptr(below), float(floor), _stream()), "heads_norm_gate")
+
+    def decayed_recurrence(self, q, k, v, log_keep, take, q_scale, state, state_slots, row_start, row_len, row_ctx, out, heads, key_heads,
+                           dim, value_dim, sums=None, totals=None):
+        n = out.shape[0]
+        rows = row_len.shape[0]
+        lib = self._part_library("recurrent")
+        if dim > lib.lsa_linear_recurrence_most_dim() or heads % key_heads:
+            raise ValueError(f"the recurrence kernel takes heads of up to {lib.lsa_linear_recurrence_most_dim()} key channels in whole groups, "
+                             f"got {dim}, {heads}/{key_heads}")
+        self._strided(q, "q", n, key_heads * dim)
+        self._strided(k, "k", n, key_heads * dim, q.dtype)
+        self._strided(v, "v", n, heads * value_dim)
+        if _code(q) and not _code(v):
+            raise TypeError("values are of the keys' type, or bfloat16 behind float32 keys")
+        _check(log_keep, "log_keep", torch.float32, (heads,) if log_keep.dim() == 1 else (n, heads))
+        if take is not None:
+            _check(take, "take", torch.float32, (n, heads))
+        _check(out, "out", torch.float32, (n, heads * value_dim))
+        for name, tensor in (("state_slots", state_slots), ("row_start", row_start), ("row_len", row_len), ("row_ctx", row_ctx)):
+            _check(tensor, name, torch.int32, (rows,))
+        if (sums is None) != (totals is None):
+            raise ValueError("the chunked recurrence takes both of its scratch tensors")
+        items = 0
+        if sums is not None:
+            items = sums.shape[0]
+            if items < n // self.MEMORY_CHUNK + rows:
+                raise ValueError(f"{items} chunks of scratch memory for {n} tokens in {rows} rows")
+            _check(sums, "sums", torch.float32, (items, heads, dim, value_dim))
+            _check(totals, "totals", torch.float32, (items, heads))
+        pointer, stride = self._state_rows(state, 0, heads * dim * value_dim, "state")
+        _launched(lib.lsa_decayed_recurrence(
+            _code(q), q.data_ptr(), q.stride(0), k.data_ptr(), k.stride(0), _code(v), v.data_ptr(), v.stride(0), _ptr(log_keep),
+            heads if log_keep.dim() == 2 else 0, _ptr(take), float(q_scale), pointer, stride, _ptr(state_slots), _ptr(row_start), _ptr(row_len),
+            _ptr(row_ctx), _ptr(out), rows, heads, heads // key_heads, dim, value_dim, _ptr(sums), _ptr(totals), items, _stream()),
+            "decayed_recurrence")
+
+    def ssd_prepare(self, x, taps, bias, state, offset, state_slots, token_row, positions, row_start, out, dt, dt_bias, a_log, steps,
+                    log_keep, keep=False):
+        n, channels = out.shape
+        count, heads, rows = taps.shape[1], steps.shape[1], row_start.shape[0]
+        if keep and n != rows:
+            raise ValueError("the state moves on inside this kernel only in steps of one token per row")
+        _check(out, "out")
+        self._strided(x, "x", n, channels, out.dtype)
+        self._strided(dt, "dt", n, heads, out.dtype)
+        _check(taps, "taps", torch.float32, (channels, count))
+        if bias is not None:
+            _check(bias, "bias", torch.float32, (channels,))
+        _check(token_row, "token_row", torch.int32, (n,))
+        _check(positions, "positions", torch.int32, (n,))
+        _check(row_start, "row_start", torch.int32)
+        _check(state_slots, "state_slots", torch.int32, (rows,))
+        _check(dt_bias, "dt_bias", torch.float32, (heads,))
+        _check(a_log, "a_log", torch.float32, (heads,))
+        _check(steps, "steps", torch.float32, (n, heads))
+        _check(log_keep, "log_keep", torch.float32, (n, heads))
+        pointer, stride = self._state_rows(state, offset, (count - 1) * channels, "state")
+        _launched(self._part_library("statespace").lsa_ssd_prepare(
+            _code(out), x.data_ptr(), x.stride(0), _ptr(taps), count, _ptr(bias), pointer, stride, _ptr(state_slots), _ptr(token_row),
+            _ptr(positions), _ptr(row_start), _ptr(out), channels, 1 if keep else 0, dt.data_ptr(), dt.stride(0), _ptr(dt_bias), _ptr(a_log),
+            _ptr(steps), _ptr(log_keep), heads, n, _stream()), "ssd_prepare")
+
+    def gated_group_norm(self, y, x, skip, gate, weight, eps, out, heads, groups):
+        n, width = out.shape
+        if width % groups or width % heads:
+            raise ValueError(f"a row of {width} does not fall into {groups} equal parts and {heads} equal heads")
+        _check(y, "y", torch.float32, (n, width))
+        _check(out, "out")
+        self._strided(x, "x", n, width, out.dtype)
+        self._strided(gate, "gate", n, width, out.dtype)
+        _check(skip, "skip", torch.float32, (heads,))
+        _check(weight, "weight", torch.float32, (width,))
+        _launched(self._part_library("statespace").lsa_gated_group_norm(
+            _code(out), _ptr(y), x.data_ptr(), x.stride(0), _ptr(skip), gate.data_ptr(), gate.stride(0), _ptr(weight), float(eps), _ptr(out),
+            groups, width // heads, width, n, _stream()), "gated_group_norm")
+
+    def rotate_heads(self, q, k, cos_sin, key_scale, out_q, out_k, heads):
+        n, width = out_q.shape
+        if width % heads:
+            raise ValueError(f"a row of {width} does not fall into {heads} equal heads")
+        self._strided(q, "q", n, width)
+        self._strided(k, "k", n, width, q.dtype)
+        _check(out_q, "out_q", torch.float32)
+        _check(out_k, "out_k", torch.float32, (n, width))
+        pairs = 0
+        if cos_sin is not None:
+            pairs = cos_sin.shape[1] // 2
+            _check(cos_sin, "cos_sin", torch.float32, (n, 2 * pairs))
+        if 2 * pairs > width // heads:
+            raise ValueError(f"{2 * pairs} dimensions turn, a head has {width // heads}")
+        _launched(self._part_library("statespace").lsa_rotate_heads(
+            _code(q), q.data_ptr(), q.stride(0), k.data_ptr(), k.stride(0), _ptr(cos_sin), pairs, float(key_scale), _ptr(out_q), _ptr(out_k),
+            heads, width // heads, n, _stream()), "rotate_heads")
 
     def scaled_sum(self, x, x_scale, y, y_scale, out):
         _check(x, "x")

@@ -13,7 +13,7 @@ from typing import Dict, Optional, Sequence
 
 import torch
 
-from ..parts.base import Block, Norm, ParamSpec, StreamUpdate
+from ..parts.base import Block, Norm, ParamSpec, Part, StreamUpdate
 from ..parts.embedding import TokenEmbedding
 from ..parts.linear import Linear
 
@@ -23,6 +23,7 @@ class LayerCall:
     block: int                  # index into ``blocks``
     cache: int                  # index of the cache this call uses
     writes_cache: bool = True   # False: read the cache another call has written
+    entry: object = None        # what happens to the stream right before this call (``forward(resid, delta, ctx, following)``), or None
 
 
 def joined(prefix: str, name: str) -> str:
@@ -32,11 +33,12 @@ def joined(prefix: str, name: str) -> str:
 
 class DecoderModel:
     """``names``: the checkpoint's names of the embedding, of the list of layers and of the final norm; layer ``i``'s
-    tensors start with ``layer_name(i)`` (default: ``<layers>.<i>``)."""
+    tensors start with ``layer_name(i)`` (default: ``<layers>.<i>``).  ``extras``: parts with tensors that belong to no layer
+    (vectors that calls of the order add to the stream), by the checkpoint's prefix."""
 
     def __init__(self, config, embedding: TokenEmbedding, blocks: Sequence[Block], final_norm: Norm, head: Linear,
                  tie_head: bool, order: Optional[Sequence[LayerCall]] = None,
-                 names=("model.embed_tokens", "model.layers", "model.norm"), layer_name=None):
+                 names=("model.embed_tokens", "model.layers", "model.norm"), layer_name=None, extras: Optional[Dict[str, Part]] = None):
         self.config = config
         self.embedding = embedding
         self.blocks = list(blocks)
@@ -46,6 +48,7 @@ class DecoderModel:
         self.order = list(order) if order is not None else [LayerCall(i, i) for i in range(len(self.blocks))]
         self.embed_name, self.layers_name, self.norm_name = names
         self.layer_name = layer_name if layer_name is not None else (lambda index: f"{self.layers_name}.{index}")
+        self.extras = dict(extras or {})
         self._owners = None
         self.after_call = None      # for whoever looks inside a step: called as (index in the order, residual, pending update) behind every call
         self.device = None
@@ -85,6 +88,9 @@ class DecoderModel:
         """(checkpoint name, owning part, the part's own name of the tensor, spec) of every tensor."""
         for k, v in self.embedding.param_specs().items():
             yield joined(self.embed_name, k), self.embedding, k, v
+        for prefix, part in self.extras.items():
+            for k, v in part.param_specs().items():
+                yield joined(prefix, k), part, k, v
         for i, block in enumerate(self.blocks):
             for k, v in block.param_specs().items():
                 yield joined(self.layer_name(i), k), block, k, v
@@ -115,7 +121,7 @@ class DecoderModel:
         if self.tie_head or not (head_names & set(assigned)):
             self.head.share_weight(self.embedding.weight)   # alias, not a copy
             self.tie_head = True
-        for part in (self.embedding, *self.blocks, self.final_norm, self.head):
+        for part in (self.embedding, *self.extras.values(), *self.blocks, self.final_norm, self.head):
             part.finalize()
         self.device, self.dtype = torch.device(device), dtype
 
@@ -130,9 +136,12 @@ class DecoderModel:
         delta = None
         for index, call in enumerate(self.order):
             block = self.blocks[call.block]
-            if block.takes_following and index + 1 < len(self.order):
+            if call.entry is not None:
+                resid, delta = call.entry.forward(resid, delta, ctx, block.entry_norm())
+            after = self.order[index + 1] if index + 1 < len(self.order) else None
+            if block.takes_following and after is not None and after.entry is None:
                 # The block may add its last update itself and prepare the next block's first norm.
-                following = self.blocks[self.order[index + 1].block].entry_norm()
+                following = self.blocks[after.block].entry_norm()
                 resid, delta = block.forward(resid, delta, ctx, caches.view(call), following=following)
             else:
                 resid, delta = block.forward(resid, delta, ctx, caches.view(call))

@@ -300,6 +300,43 @@ class HyperConnection(Part):
         self.read, self.mix = self.read.contiguous(), self.mix.contiguous()
 
 
+class LoopSteps(Part):
+    """The vectors that join the stream in front of the passes over a run of layers, one a pass: ``[times, width]``."""
+
+    def __init__(self, times: int, width: int, tensor: str = "step"):
+        self.times, self.width, self.tensor = int(times), int(width), tensor
+        self.vectors = None
+
+    def param_specs(self):
+        return {self.tensor: ParamSpec((self.times, self.width), VECTOR, "bias", share_per_token=1.0 / self.times)}
+
+    def assign(self, name, tensor):
+        if name != self.tensor:
+            raise KeyError(name)
+        self.vectors = tensor.contiguous()
+
+
+class PassEntry:
+    """What happens to the stream in front of pass ``number`` over a run of layers: the embedding's output is added again
+    (every pass but the first), then the pass's vector; the next block's first norm is carried out on the way.  The stream
+    is one of 32-bit, ``[1, T, W]``, to which everything has been added."""
+
+    def __init__(self, steps: LoopSteps, number: int, embedding):
+        self.steps, self.number, self.embedding = steps, int(number), embedding
+
+    def forward(self, resid, delta, ctx, following=None):
+        """``(stream, update)`` as a block hands them on, the update telling that ``following`` has been carried out."""
+        if isinstance(delta, StreamUpdate):
+            resid, delta = delta.resid, None
+        if delta is not None or resid.dim() != 3 or resid.shape[0] != 1:
+            raise ValueError("a pass over layers begins on one 32-bit stream to which everything has been added")
+        normed = ctx.empty(resid.shape[1:]) if following is not None else None
+        ctx.ops.stream_inject(resid[0], self.embedding.weight, ctx.token_ids, self.embedding.scale if self.number else 0.0,
+                              self.steps.vectors[self.number], following.weight if following is not None else None,
+                              following.eps if following is not None else 0.0, normed)
+        return resid, (StreamUpdate(following, resid, normed=normed) if normed is not None else None)
+
+
 class MultiStreamBlock(Block):
     """Pre-norm sublayers over several residual streams kept in 32-bit, ``[streams, T, W]``: each sublayer reads a
     weighted sum of the streams under its norm and writes its result, times a constant, back into all of them through

@@ -37,7 +37,8 @@ class KernelNamespace:
     def add_bias_(self, y, bias):
         raise NotImplementedError
 
-    def rotary_table(self, positions, inv_freq):
+    def rotary_table(self, positions, inv_freq, amplitude=1.0):
+        """float32 ``[T, 2 * len(inv_freq)]``: the cosines, then the sines, of ``position * inv_freq``, all times ``amplitude``."""
         raise NotImplementedError
 
     def qk_norm_rope_kv_write(self, qkv, keys, values, table, token_row, positions, q_weight, k_weight, eps, cos_sin,
@@ -95,7 +96,7 @@ class KernelNamespace:
 
     def heads_norm_gate(self, x, weight, weight_per_channel, eps, gate, out, heads, value_dim, gate_activation="silu", below=None, floor=0.0):
         """``out[t, h, :] = x'[t, h, :] / rms(x'[t, h, :]) * w * act(gate[t, h, :])``; ``x`` float32, ``w = weight [value_dim]``
-        shared by the heads or, with ``weight_per_channel``, ``weight [heads * value_dim]``; ``gate`` a view like ``out``;
+        shared by the heads or, with ``weight_per_channel``, ``weight [heads * value_dim]`` (None: 1); ``gate`` a view like ``out``;
         ``act``: ``"silu"`` or ``"sigmoid"``.  ``x' = x``, or, with ``below [T, heads, 2]`` (float32):
         ``x / (max(|below[..., 0]|, below[..., 1]) + floor)``, a matrix memory's read-out under its normaliser."""
         raise NotImplementedError
@@ -118,6 +119,43 @@ class KernelNamespace:
         the slot holds; the state after the row's last token is stored back.  ``run`` (float64 ``[T, heads]``) and ``sums``
         (float32 ``[chunks, heads, dim, value_dim + 1]``): scratch memory of the chunked form, given when
         ``matrix_memory_chunks`` said so."""
+        raise NotImplementedError
+
+    # Recurrences with one decay per head, and what state-space mixers and retention have around them.
+    def decayed_recurrence(self, q, k, v, log_keep, take, q_scale, state, state_slots, row_start, row_len, row_ctx, out, heads, key_heads,
+                           dim, value_dim, sums=None, totals=None):
+        """Per row (request) and head, over the row's tokens in order, all float32: ``S_t = exp(log_keep_t) S_(t-1) + take_t
+        k_t v_t^T``, ``out_t = S_t^T (q_t * q_scale)``.  ``log_keep [T, heads]``, or ``[heads]``: the same for every token;
+        ``take [T, heads]``, or None: 1.  ``q, k [T, key_heads * dim]``, ``v [T, heads * value_dim]`` (views with unit stride along a
+        row; head ``h`` reads query and key head ``h // (heads / key_heads)``), ``out [T, heads * value_dim]`` float32.
+        ``S [heads, dim, value_dim]`` lies at the front of ``state[slot]``; a row whose first token stands at position 0 starts
+        from zeros whatever the slot holds; the state after the row's last token is stored back.  ``sums`` (float32 ``[chunks,
+        heads, dim, value_dim]``) and ``totals`` (float32 ``[chunks, heads]``): scratch memory of the chunked form, given when
+        ``matrix_memory_chunks`` said so."""
+        raise NotImplementedError
+
+    def ssd_prepare(self, x, taps, bias, state, offset, state_slots, token_row, positions, row_start, out, dt, dt_bias, a_log, steps,
+                    log_keep, keep=False):
+        """``out [T, C] = silu(bias + conv(x))`` of ``x``'s type: a causal convolution over each request's tokens per channel
+        (``taps [C, K]``, tap ``j`` on the token ``K - 1 - j`` places back, zeros before the sequence, earlier steps' inputs from
+        ``state[slot, offset:]`` as ``[K - 1, C]``, oldest first).  Beside it ``steps [T, heads] = softplus(dt + dt_bias)`` and
+        ``log_keep = -exp(a_log) * steps``, float32.  ``keep`` (steps of one token per row only): the state also moves on by the
+        step's token, as :meth:`delta_conv_keep` would do."""
+        raise NotImplementedError
+
+    def gated_group_norm(self, y, x, skip, gate, weight, eps, out, heads, groups):
+        """``u = (y + skip[head] * x) * silu(gate)``, ``out = u / rms(u) * weight`` with a root mean square for each of ``groups``
+        equal parts of a row; ``y [T, width]`` float32, ``x``, ``gate`` views of ``out``'s type, ``skip [heads]``, ``weight [width]``."""
+        raise NotImplementedError
+
+    def rotate_heads(self, q, k, cos_sin, key_scale, out_q, out_k, heads):
+        """Every head's first ``2 * pairs`` dimensions turn, ``i`` with ``i + pairs``, by ``cos_sin [T, 2 * pairs]`` (None: nothing
+        turns); keys are then multiplied by ``key_scale``.  ``q, k`` views of one type, results float32."""
+        raise NotImplementedError
+
+    def stream_inject(self, x, table, token_ids, scale, vector, next_weight=None, next_eps=0.0, normed=None):
+        """``x [T, W] += table[token_ids] * scale + vector`` in float32, where it lies (``scale`` 0: the vector only); with
+        ``next_weight``: ``normed = rmsnorm(x) * next_weight`` (eps ``next_eps``, any type)."""
         raise NotImplementedError
 
     # Several residual streams in 32-bit.
@@ -181,12 +219,13 @@ class KernelNamespace:
 
     # Attention over a shared low-rank latent.
     def latent_prepare(self, proj, q_latent, norm_weight, eps, cos_sin, keys, values, table, token_row, positions, page_size,
-                       out_q, n_heads, dim, rot_dim, rank, write_cache=True, up_keys=None):
+                       out_q, n_heads, dim, rot_dim, rank, write_cache=True, up_keys=None, pairing="neighbours"):
         """``proj [T, n_heads * (dim + rot_dim) + rank + rot_dim + ...]``: per head ``dim`` plain and ``rot_dim`` rotated
         query dimensions, then the token's ``rank`` latent dimensions and its ``rot_dim`` shared rotated key dimensions.
         Writes a cache row ``[rmsnorm(latent) * norm_weight, rotate(key part), zeros]`` of every token as its key and,
         transposed, as its value, and ``out_q [T, n_heads * D]`` with per head ``[q_latent[h, t], rotate(q's rotated part),
-        zeros]``.  ``cos_sin [T, 2 * pairs]``: neighbouring dimensions (2i, 2i+1) of the first ``2 * pairs`` rotated ones turn.
+        zeros]``.  ``cos_sin [T, 2 * pairs]``: neighbouring dimensions (2i, 2i+1) of the first ``2 * pairs`` rotated ones turn together,
+        or, with ``pairing="halves"``, dimensions i and i + pairs.
         ``q_latent`` None and ``up_keys [heads, dim, rank]`` given: ``q_latent[h, t] = q_plain[t, h] @ up_keys[h]`` is made here."""
         raise NotImplementedError
 
@@ -239,20 +278,28 @@ class KernelNamespace:
         raise NotImplementedError
 
     # Routed experts.
-    def route_experts(self, x, router, top, chosen, weights, scoring="softmax", groups=None, bias=None):
+    def route_experts(self, x, router, top, chosen, weights, scoring="softmax", groups=None, bias=None, correction=None, weight_scale=1.0,
+                      gate_out=None):
         """Float32 logits ``x router^T``; ``chosen [T, top]`` the largest (first of equals), ``weights`` their softmax.
         ``scoring="sigmoid"``: scores ``sigmoid(logits)``, the largest scores chosen, the scores themselves the weights;
         ``groups=(count, keep)``: only experts of the ``keep`` best of ``count`` equal groups of neighbours can be chosen,
-        a group's score the sum of its two largest scores (the first of equal groups).  ``bias [experts]`` joins the logits."""
+        a group's score the sum of its two largest scores (the first of equal groups).  ``bias [experts]`` joins the logits.
+        ``scoring="softmax_all"``: scores are the softmax over all experts; the largest of ``score + correction`` (``[experts]`` or
+        None) are chosen; the weights are the chosen scores divided by (their sum + 1e-20), times ``weight_scale``.
+        ``gate_out [T]``: ``router`` has one more row, a gate of one number a token: its logit's sigmoid."""
         raise NotImplementedError
 
-    def experts_gate_up(self, x, gate_up, chosen, hidden, activation="silu", limit=0.0):
+    def experts_gate_up(self, x, gate_up, chosen, hidden, activation="silu", limit=0.0, identity=0, shared=None):
         """``hidden[t * top + s] = silu(G x_t) * (U x_t)`` with ``[G; U] = gate_up[chosen[t, s]]`` (``[E, 2F, W]``);
-        ``activation="clamped"``: ``g = min(G x, limit)``, ``u = clamp(U x, -limit, limit)``, ``g * sigmoid(1.702 g) * (u + 1)``."""
+        ``activation="clamped"``: ``g = min(G x, limit)``, ``u = clamp(U x, -limit, limit)``, ``g * sigmoid(1.702 g) * (u + 1)``.
+        ``identity``: that many choices from ``E`` on are identity experts, with nothing to multiply.  ``shared = (gate_up [2F', W],
+        hidden [T, F'])``: the shared expert's hidden rows are made beside the others."""
         raise NotImplementedError
 
-    def experts_down(self, hidden, down, chosen, weights, out):
-        """``out[t] = sum_s weights[t, s] * down[chosen[t, s]] hidden[t * top + s]``; ``down [E, W, F]``, ``out`` float32."""
+    def experts_down(self, hidden, down, chosen, weights, out, x=None, shared=None, shared_y=None, shared_gate=None):
+        """``out[t] = sum_s weights[t, s] * down[chosen[t, s]] hidden[t * top + s]``; ``down [E, W, F]``, ``out`` float32.
+        ``x [T, W]`` given: choices from ``E`` on are identity experts, whose output is ``x[t]``.  ``shared_gate [T]``: the shared
+        expert's output, ``shared_y [T, W]`` or ``shared = (down [W, F'], hidden [T, F'])``, joins times the gate."""
         raise NotImplementedError
 
     def sample(self, logits, temperature, uniform, out):
@@ -264,10 +311,16 @@ class KernelNamespace:
         products themselves (``up_keys=`` / ``up_values=``) instead of getting them from batched products made before."""
         return False
 
-    def experts_sorted(self, x, gate_up, down, chosen, weights, out, activation="silu", limit=0.0) -> bool:
+    def experts_sorted(self, x, gate_up, down, chosen, weights, out, activation="silu", limit=0.0, identity=0, shared_y=None,
+                       shared_gate=None) -> bool:
         """Both products of the routed experts and the weighted sum for all of the step's tokens at once, the (token,
         expert) pairs sorted by expert so that an expert's matrices are read once per tile of pairs: ``out`` as
         :meth:`experts_down` leaves it.  False: not done (not offered, or it would not pay for these sizes)."""
+        return False
+
+    def shared_expert_inside(self, n_tokens: int) -> bool:
+        """Whether, for a step of this many tokens, :meth:`experts_gate_up` and :meth:`experts_down` should make the shared expert's
+        products themselves instead of getting its output from products of its own."""
         return False
 
     def check_cache_geometry(self, cache_specs, page_size: int, num_pages=None) -> None:

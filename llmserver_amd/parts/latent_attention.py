@@ -49,8 +49,8 @@ class LatentAttention(Mixer):
                  gate_per_channel: bool = False):
         """``window``: a query sees itself and the ``window - 1`` positions before it (None: all).  ``gate_per_channel``:
         the gate's projection has a row for every channel of every head's values instead of one a head."""
-        if getattr(position, "pairing", None) != "neighbours":
-            raise ValueError("this mixer's kernels turn neighbouring dimensions together; it takes a PairedRotaryPosition")
+        if getattr(position, "pairing", None) not in ("neighbours", "halves"):
+            raise ValueError("this mixer's kernels turn dimensions together as neighbours or as halves; it takes a rotary position")
         if position.rotary_dim is None or position.rotary_dim > rot_dim or position.rotary_dim % 2:
             raise ValueError(f"the position encoding turns {position.rotary_dim} dimensions, the rotated part has {rot_dim}")
         self.width, self.n_heads, self.dim, self.rot_dim, self.value_dim, self.rank = width, n_heads, dim, rot_dim, value_dim, rank
@@ -143,7 +143,8 @@ class LatentAttention(Mixer):
         q = ctx.empty((n, self.n_heads * self.row))
         ops.latent_prepare(proj, q_latent, self.down_norm_weight, self.norm_eps, self.position.cos_sin(ctx), cache.keys, cache.values,
                            table, ctx.token_row, ctx.positions, cache.page_size, q, self.n_heads, self.dim, self.rot_dim, self.rank,
-                           cache.writable, **({"up_keys": self.up_keys} if inside else {}))
+                           cache.writable, **({"up_keys": self.up_keys} if inside else {}),
+                         **({"pairing": "halves"} if self.position.pairing == "halves" else {}))
         mixed = ctx.empty((n, self.n_heads * self.row))
         extra = {"sinks": self.sinks} if self.sinks is not None else {}
         ops.paged_attention(q, mixed, cache.keys, cache.values, table, ctx.row_start, ctx.row_len, ctx.row_ctx,

@@ -121,9 +121,9 @@ class TorchOps(KernelNamespace):
     def add_bias_(self, y, bias):
         y.copy_((y.float() + bias).to(y.dtype))
 
-    def rotary_table(self, positions, inv_freq):
+    def rotary_table(self, positions, inv_freq, amplitude=1.0):
         angles = positions.float()[:, None] * inv_freq[None, :]
-        return torch.cat([torch.cos(angles), torch.sin(angles)], dim=1)
+        return amplitude * torch.cat([torch.cos(angles), torch.sin(angles)], dim=1)
 
     def qk_norm_rope_kv_write(self, qkv, keys, values, table, token_row, positions, q_weight, k_weight, eps, cos_sin,
                               page_size, n_q, n_kv, head_dim, write_cache=True):
@@ -382,7 +382,8 @@ class TorchOps(KernelNamespace):
         if below is not None:
             rows = rows / (torch.maximum(below[..., 0].abs(), below[..., 1]) + floor)[..., None]
         normed = self._rms(rows, eps)
-        normed = normed * (weight.view(heads, value_dim) if weight_per_channel else weight)
+        if weight is not None:
+            normed = normed * (weight.view(heads, value_dim) if weight_per_channel else weight)
         g = gate.float().reshape(n, heads, value_dim)
         g = torch.sigmoid(g) if gate_activation == "sigmoid" else g * torch.sigmoid(g)
         out.copy_((normed * g).reshape(n, heads * value_dim).to(out.dtype))
@@ -420,6 +421,76 @@ class TorchOps(KernelNamespace):
             state[slot, matrix_size:matrix_size + normaliser_size] = normaliser.reshape(-1)
             state[slot, matrix_size + normaliser_size:matrix_size + normaliser_size + heads] = top
 
+    # -- recurrences with one decay per head ---------------------------------------------------------------
+    def decayed_recurrence(self, q, k, v, log_keep, take, q_scale, state, state_slots, row_start, row_len, row_ctx, out, heads, key_heads,
+                           dim, value_dim, sums=None, totals=None):
+        assert sums is None and totals is None
+        n, size, each = out.shape[0], heads * dim * value_dim, heads // key_heads
+        keep = torch.exp(log_keep).expand(n, heads)
+        for row in range(len(row_len)):
+            start, count, end = int(row_start[row]), int(row_len[row]), int(row_ctx[row])
+            if count <= 0:
+                continue
+            slot = int(state_slots[row])
+            matrix = state[slot, :size].view(heads, dim, value_dim).clone()
+            if end - count == 0:
+                matrix.zero_()
+            for t in range(start, start + count):
+                qt = q[t].float().view(key_heads, dim).repeat_interleave(each, dim=0) * q_scale
+                kt = k[t].float().view(key_heads, dim).repeat_interleave(each, dim=0)
+                vt = v[t].float().view(heads, value_dim) * (1.0 if take is None else take[t][:, None])
+                matrix = keep[t][:, None, None] * matrix + kt[:, :, None] * vt[:, None, :]
+                out[t] = torch.einsum("hdv,hd->hv", matrix, qt).reshape(-1)
+            state[slot, :size] = matrix.reshape(-1)
+
+    def ssd_prepare(self, x, taps, bias, state, offset, state_slots, token_row, positions, row_start, out, dt, dt_bias, a_log, steps,
+                    log_keep, keep=False):
+        steps.copy_(torch.nn.functional.softplus(dt.float() + dt_bias))
+        log_keep.copy_(-torch.exp(a_log) * steps)
+        channels, count = taps.shape
+        kept, wide = count - 1, x.float()
+        result = torch.zeros_like(wide) + (0.0 if bias is None else bias)
+        for t in range(wide.shape[0]):
+            row, position = int(token_row[t]), int(positions[t])
+            first = position - (t - int(row_start[row]))
+            old = state[int(state_slots[row]), offset:offset + kept * channels].view(kept, channels)
+            for j in range(count):
+                place = position - (kept - j)
+                if place >= 0:
+                    result[t] += taps[:, j] * (wide[t - (kept - j)] if place >= first else old[kept - (first - place)])
+        out.copy_((result * torch.sigmoid(result)).to(out.dtype))
+        if keep and kept:
+            assert wide.shape[0] == len(row_start)
+            for t in range(wide.shape[0]):
+                slot = int(state_slots[int(token_row[t])])
+                old = state[slot, offset:offset + kept * channels].view(kept, channels)
+                state[slot, offset:offset + kept * channels] = torch.cat([old[1:], wide[t:t + 1]], dim=0).reshape(-1)
+
+    def gated_group_norm(self, y, x, skip, gate, weight, eps, out, heads, groups):
+        n, width = out.shape
+        z = gate.float()
+        u = (y.view(n, heads, -1) + skip[:, None] * x.float().reshape(n, heads, -1)).reshape(n, width) * (z * torch.sigmoid(z))
+        out.copy_((self._rms(u.view(n, groups, -1), eps).reshape(n, width) * weight).to(out.dtype))
+
+    def rotate_heads(self, q, k, cos_sin, key_scale, out_q, out_k, heads):
+        n = out_q.shape[0]
+
+        def turned(x):
+            x = x.float().reshape(n, heads, -1)
+            if cos_sin is None:
+                return x
+            pairs = cos_sin.shape[1] // 2
+            c, s = cos_sin[:, None, :pairs], cos_sin[:, None, pairs:]
+            u, v = x[..., :pairs], x[..., pairs:2 * pairs]
+            return torch.cat([u * c - v * s, v * c + u * s, x[..., 2 * pairs:]], dim=-1)
+        out_q.copy_(turned(q).reshape(n, -1))
+        out_k.copy_((turned(k) * key_scale).reshape(n, -1))
+
+    def stream_inject(self, x, table, token_ids, scale, vector, next_weight=None, next_eps=0.0, normed=None):
+        x += (table[token_ids.long()].float() * scale if scale else 0.0) + vector
+        if next_weight is not None:
+            normed.copy_((self._rms(x, next_eps) * next_weight).to(normed.dtype))
+
     def scaled_sum(self, x, x_scale, y, y_scale, out):
         out.copy_((x_scale * x.float() + y_scale * y.float()).to(out.dtype))
 
@@ -430,7 +501,7 @@ class TorchOps(KernelNamespace):
         return self.inside
 
     def latent_prepare(self, proj, q_latent, norm_weight, eps, cos_sin, keys, values, table, token_row, positions, page_size,
-                       out_q, n_heads, dim, rot_dim, rank, write_cache=True, up_keys=None):
+                       out_q, n_heads, dim, rot_dim, rank, write_cache=True, up_keys=None, pairing="neighbours"):
         n, width = proj.shape[0], keys.shape[-1]
         q = proj[:, :n_heads * (dim + rot_dim)].float().view(n, n_heads, dim + rot_dim)
         if q_latent is None:
@@ -441,8 +512,11 @@ class TorchOps(KernelNamespace):
 
         def turned(x):                                  # x [T, ..., rot_dim]
             shape = [n] + [1] * (x.dim() - 2) + [pairs]
-            u, v = x[..., 0:2 * pairs:2], x[..., 1:2 * pairs:2]
             c, s = cos.view(shape), sin.view(shape)
+            if pairing == "halves":
+                u, v = x[..., :pairs], x[..., pairs:2 * pairs]
+                return torch.cat([u * c - v * s, v * c + u * s, x[..., 2 * pairs:]], dim=-1)
+            u, v = x[..., 0:2 * pairs:2], x[..., 1:2 * pairs:2]
             return torch.cat([torch.stack([u * c - v * s, v * c + u * s], dim=-1).flatten(-2), x[..., 2 * pairs:]], dim=-1)
 
         full = torch.zeros((n, n_heads, width), dtype=torch.float32, device=proj.device)
@@ -572,10 +646,29 @@ class TorchOps(KernelNamespace):
             state[slot, offset:offset + size] = kept.view(heads, dim, blocks, 16).permute(0, 2, 1, 3).reshape(-1)
 
     # -- routed experts ----------------------------------------------------------------------------------
-    def route_experts(self, x, router, top, chosen, weights, scoring="softmax", groups=None, bias=None):
+    inside_shared = False          # True: the parts are told to have the shared expert's products made beside the routed experts'
+
+    def shared_expert_inside(self, n_tokens):
+        return self.inside_shared
+
+    def route_experts(self, x, router, top, chosen, weights, scoring="softmax", groups=None, bias=None, correction=None, weight_scale=1.0,
+                      gate_out=None):
         logits = x.float() @ router.float().t()
+        if gate_out is not None:
+            gate_out.copy_(torch.sigmoid(logits[:, -1]))
+            logits = logits[:, :-1]
         if bias is not None:
             logits = logits + bias
+        if scoring == "softmax_all":
+            scores = torch.softmax(logits, dim=-1)
+            values = scores if correction is None else scores + correction
+            for k in range(top):                                # the largest values, the first of equal ones
+                pick = values.argmax(dim=-1, keepdim=True)
+                chosen[:, k] = pick[:, 0].to(chosen.dtype)
+                weights[:, k] = scores.gather(1, pick)[:, 0]
+                values = values.scatter(1, pick, float("-inf"))
+            weights.copy_(weights / (weights.sum(dim=-1, keepdim=True) + 1e-20) * weight_scale)
+            return
         if scoring == "softmax":
             best = torch.topk(logits, top, dim=-1)
             chosen.copy_(best.indices.to(chosen.dtype))
@@ -599,10 +692,17 @@ class TorchOps(KernelNamespace):
             weights[:, k] = scores.gather(1, pick)[:, 0]
             allowed = allowed.scatter(1, pick, float("-inf"))
 
-    def experts_gate_up(self, x, gate_up, chosen, hidden, activation="silu", limit=0.0):
+    def experts_gate_up(self, x, gate_up, chosen, hidden, activation="silu", limit=0.0, identity=0, shared=None):
         top, inter = chosen.shape[1], hidden.shape[1]
+        if shared is not None:
+            both = x.float() @ shared[0].float().t()
+            gate, up = both[:, :both.shape[1] // 2], both[:, both.shape[1] // 2:]
+            shared[1].copy_((self._activated(gate, activation) * up).to(x.dtype))
         for t in range(x.shape[0]):
             for s in range(top):
+                if identity and int(chosen[t, s]) >= gate_up.shape[0]:
+                    hidden[t * top + s] = float("nan")          # (nobody reads it)
+                    continue
                 both = gate_up[int(chosen[t, s])].float() @ x[t].float()
                 gate, up = both[:inter], both[inter:]
                 if activation == "clamped":
@@ -611,11 +711,18 @@ class TorchOps(KernelNamespace):
                 else:
                     hidden[t * top + s] = (gate * torch.sigmoid(gate) * up).to(hidden.dtype)
 
-    def experts_down(self, hidden, down, chosen, weights, out):
+    def experts_down(self, hidden, down, chosen, weights, out, x=None, shared=None, shared_y=None, shared_gate=None):
         top = chosen.shape[1]
         out.zero_()
+        if shared is not None:
+            shared_y = shared[1].float() @ shared[0].float().t()
+        if shared_gate is not None:
+            out += shared_gate[:, None] * shared_y.float()
         for t in range(out.shape[0]):
             for s in range(top):
+                if x is not None and int(chosen[t, s]) >= down.shape[0]:
+                    out[t] += weights[t, s] * x[t].float()
+                    continue
                 out[t] += weights[t, s] * (down[int(chosen[t, s])].float() @ hidden[t * top + s].float())
 
     def sample(self, logits, temperature, uniform, out):
