@@ -130,6 +130,30 @@ NAMED_SIZES.update({
 })
 
 
+def _setodra(width, heads, dim, rot_dim, kv_rank, retention_heads, retention_dim, retention_vdim, ssd_heads, ssd_vdim, ssd_state, ssd_groups, ff, experts,
+             top, identity, vocab=32768):
+    space = ("mamba2", {"heads": ssd_heads, "vdim": ssd_vdim, "state": ssd_state, "groups": ssd_groups, "conv": 4, "norm_groups": ssd_groups})
+    latent = ("latent_attention", {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": dim, "kv_rank": kv_rank, "scale": (dim + rot_dim) ** -0.5,
+                                   "rot": {"base": 10000.0, "dims": rot_dim,
+                                           "scaling": {"factor": 8.0, "original": 4096.0, "fast": 32.0, "slow": 1.0}}})
+    retention = ("retention", {"heads": retention_heads, "dim": retention_dim, "vdim": retention_vdim, "rot": {"base": 10000.0, "dims": retention_dim},
+                               "decay": [1.0 - 2.0 ** (-5.0 - index % 8) for index in range(retention_heads)]})
+    mlp = {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "top": top, "scale": 1.0, "identity": identity}, "shared": {"ff": ff}}
+    return {"architecture": "Setodra", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0},
+            "loop": {"start": 2, "stop": 4, "times": 2},
+            "layers": [{"type": kind, "mixer": dict(mixer), "mlp": dict(mlp)} for kind, mixer in (space, latent, retention, space, latent, space)]}
+
+
+# Setodra at the widths of the sizes above: six layers, the two in the middle passed twice, so eight runs: four state-space
+# mixers of 64 (128) heads with values of 64, a state of 128 and 8 groups (a state of 2 MB (4 MB) a run and request), two of
+# latent attention of the Zepolix sizes' shape with a stretched rotation, two retentions of the shape of the Kerudra sizes' memories;
+# experts of the Zepolix sizes' shape with one identity expert for every eight and a shared expert of the same size.
+NAMED_SIZES.update({
+    "setodra-2k": _setodra(2048, 16, 128, 64, 192, 8, 128, 256, 64, 64, 128, 8, 1408, 64, 6, 8),
+    "setodra-4k": _setodra(4096, 32, 128, 64, 192, 16, 128, 256, 128, 64, 128, 8, 2048, 32, 4, 4),
+})
+
+
 def named_size(name: str) -> dict:
     """The entry's keys, a copy the caller may change (fewer layers, say)."""
     try:
@@ -149,6 +173,8 @@ def with_layers(raw: dict, layers: Optional[int]) -> dict:
     if layers:
         if isinstance(raw.get("layers"), list):
             raw["layers"] = raw["layers"][:int(layers)]
+            if raw.get("loop") and raw["loop"]["stop"] > len(raw["layers"]):
+                del raw["loop"]                      # (a pass over layers that are not all there)
         else:
             raw["num_hidden_layers"] = min(int(raw["num_hidden_layers"]), int(layers))
     return raw

@@ -69,21 +69,24 @@ __device__ inline void wave_dot2(const T* __restrict__ w0, const T* __restrict__
 }
 
 // Router logits for steps of few tokens, where a library product would be a launch of 11 us for a few thousand
-// multiplications: grid (tokens, experts / 4), a wavefront per expert, float32 throughout.
-__global__ __launch_bounds__(256) void route_logits_kernel(const float* __restrict__ x, const float* __restrict__ router,
+// multiplications: grid (tokens, experts / 4), a wavefront per expert; the rows are widened as they are read, the rest is float32.
+template <typename T>
+__global__ __launch_bounds__(256) void route_logits_kernel(const T* __restrict__ x, const float* __restrict__ router,
                                                            float* __restrict__ logits, int experts, int width) {
     const int lane = threadIdx.x & 63, e = blockIdx.y * 4 + (threadIdx.x >> 6), t = blockIdx.x;
     if (e >= experts) return;
     const float* r = router + (size_t)e * width;
-    const float* row = x + (size_t)t * width;
+    const T* row = x + (size_t)t * width;
     float acc = 0.f;
     if (width % 4 == 0) {
+        struct alignas(4 * sizeof(T)) Four { T v[4]; };
         for (int i = lane * 4; i < width; i += 256) {
-            const float4 a = *reinterpret_cast<const float4*>(r + i), b = *reinterpret_cast<const float4*>(row + i);
-            acc += a.x * b.x + a.y * b.y + a.z * b.z + a.w * b.w;
+            const float4 a = *reinterpret_cast<const float4*>(r + i);
+            const Four b = *reinterpret_cast<const Four*>(row + i);
+            acc += a.x * (float)b.v[0] + a.y * (float)b.v[1] + a.z * (float)b.v[2] + a.w * (float)b.v[3];
         }
     } else {
-        for (int i = lane; i < width; i += 64) acc += r[i] * row[i];
+        for (int i = lane; i < width; i += 64) acc += r[i] * (float)row[i];
     }
     acc = wave_sum(acc);
     if (lane == 0) logits[(size_t)t * experts + e] = acc;
@@ -110,22 +113,29 @@ __global__ __launch_bounds__(256) void route_top_kernel(const float* __restrict_
     float* scores = logits + experts;
     const bool sigmoid_scores = scoring == 1;
     if (gate_out && lane == 0) gate_out[t] = 1.f / (1.f + expf(-all_logits[(size_t)t * stride + experts]));
-    float most = 0.f, all = 1.f;
-    if (scoring == 2) {                                        // the softmax over all experts
-        most = NEG_INF;
-        for (int e = lane; e < experts; e += 64) most = fmaxf(most, all_logits[(size_t)t * stride + e] + (bias ? bias[e] : 0.f));
-        most = wave_max(most);
-        all = 0.f;
-        for (int e = lane; e < experts; e += 64) all += expf(all_logits[(size_t)t * stride + e] + (bias ? bias[e] : 0.f) - most);
-        all = wave_sum(all);
-    }
+    float most = NEG_INF;
     for (int e = lane; e < experts; e += 64) {
         float v = all_logits[(size_t)t * stride + e];
         if (bias) v += bias[e];                            // (a bias per expert joins the logits)
+        most = fmaxf(most, v);
         if (sigmoid_scores) v = 1.f / (1.f + expf(-v));
-        if (scoring == 2) v = expf(v - most) / all;
         scores[e] = v;
-        logits[e] = correction ? v + correction[e] : v;
+        logits[e] = v;
+    }
+    if (scoring == 2) {                                    // the softmax over all experts (a lane meets its own entries only)
+        most = wave_max(most);
+        float all = 0.f;
+        for (int e = lane; e < experts; e += 64) {
+            const float v = expf(scores[e] - most);
+            scores[e] = v;
+            all += v;
+        }
+        all = wave_sum(all);
+        for (int e = lane; e < experts; e += 64) {
+            const float v = scores[e] / all;
+            scores[e] = v;
+            logits[e] = correction ? v + correction[e] : v;
+        }
     }
     __builtin_amdgcn_wave_barrier();
     if (sigmoid_scores && groups > 1) {
@@ -328,9 +338,11 @@ __global__ __launch_bounds__(256) void experts_down_kernel(const T* __restrict__
     }
 }
 
-LSA_EXPORT int lsa_route_logits(const float* x, const float* router, float* logits, int n, int experts, int width, hipStream_t stream) {
+LSA_EXPORT int lsa_route_logits(int code, const void* x, const float* router, float* logits, int n, int experts, int width, hipStream_t stream) {
     if (n <= 0) return 0;
-    route_logits_kernel<<<dim3(n, (experts + 3) / 4), 256, 0, stream>>>(x, router, logits, experts, width);
+    const dim3 grid(n, (experts + 3) / 4);
+    if (code) route_logits_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)x, router, logits, experts, width);
+    else route_logits_kernel<float><<<grid, 256, 0, stream>>>((const float*)x, router, logits, experts, width);
     LSA_LAUNCH_CHECK();
 }
 
@@ -551,32 +563,46 @@ __global__ __launch_bounds__(256) void experts_tile_kernel(const bf16_t* __restr
 }
 
 // out[t][c] = sum_s weights[t][s] * y[t * top + s][c]; with `beside`: identity experts (choices from `experts` on) put the token's
-// row in place of y, and the shared expert's output joins times the token's gate.
+// row in place of y, and the shared expert's output joins times the token's gate.  grid (tokens, blocks of 256 V columns), a
+// thread has V neighbouring columns of one token.
+template <int V>
 __global__ __launch_bounds__(256) void experts_combine_kernel(const float* __restrict__ y, const float* __restrict__ weights,
                                                               float* __restrict__ out, int top, int width, const int* __restrict__ chosen,
                                                               int experts, BesideExperts<bf16_t> beside) {
-    const int t = blockIdx.x;
-    if (beside.x || beside.gate) {
-        const float gate = beside.gate ? beside.gate[t] : 0.f;
-        float identity_weight = 0.f;
-        if (beside.x)
-            for (int s = 0; s < top; ++s)
-                if (chosen[(size_t)t * top + s] >= experts) identity_weight += weights[(size_t)t * top + s];
-        for (int c = threadIdx.x; c < width; c += blockDim.x) {
-            float acc = 0.f;
-            for (int s = 0; s < top; ++s)
-                if (!beside.x || chosen[(size_t)t * top + s] < experts) acc += weights[(size_t)t * top + s] * y[((size_t)t * top + s) * width + c];
-            if (beside.gate) acc += gate * (float)beside.y[(size_t)t * width + c];
-            if (beside.x) acc += identity_weight * (float)beside.x[(size_t)t * width + c];
-            out[(size_t)t * width + c] = acc;
+    struct alignas(4 * V) Floats { float v[V]; };
+    struct alignas(2 * V) Halves { bf16_t v[V]; };
+    const int t = blockIdx.x, c = (blockIdx.y * 256 + threadIdx.x) * V;
+    if (c >= width) return;
+    float acc[V];
+#pragma unroll
+    for (int v = 0; v < V; ++v) acc[v] = 0.f;
+    if (beside.gate) {
+        const Halves h = *reinterpret_cast<const Halves*>(beside.y + (size_t)t * width + c);
+        const float gate = beside.gate[t];
+#pragma unroll
+        for (int v = 0; v < V; ++v) acc[v] = gate * (float)h.v[v];
+    }
+    float identity_weight = 0.f;
+#pragma unroll 4
+    for (int s = 0; s < top; ++s) {                          // (choice and weight are the same for the whole workgroup)
+        const float weight = weights[(size_t)t * top + s];
+        if (beside.x && chosen[(size_t)t * top + s] >= experts) {
+            identity_weight += weight;
+            continue;
         }
-        return;
+        const Floats f = *reinterpret_cast<const Floats*>(y + ((size_t)t * top + s) * width + c);
+#pragma unroll
+        for (int v = 0; v < V; ++v) acc[v] += weight * f.v[v];
     }
-    for (int c = threadIdx.x; c < width; c += blockDim.x) {
-        float acc = 0.f;
-        for (int s = 0; s < top; ++s) acc += weights[(size_t)t * top + s] * y[((size_t)t * top + s) * width + c];
-        out[(size_t)t * width + c] = acc;
+    if (beside.x) {
+        const Halves h = *reinterpret_cast<const Halves*>(beside.x + (size_t)t * width + c);
+#pragma unroll
+        for (int v = 0; v < V; ++v) acc[v] += identity_weight * (float)h.v[v];
     }
+    Floats result;
+#pragma unroll
+    for (int v = 0; v < V; ++v) result.v[v] = acc[v];
+    *reinterpret_cast<Floats*>(out + (size_t)t * width + c) = result;
 }
 
 LSA_EXPORT int lsa_experts_tile_rows() { return TILE_M; }
@@ -611,7 +637,7 @@ LSA_EXPORT int lsa_experts_tiled(const void* x, const void* gate_up, const void*
         else LSA_TILES(32, 4);
     }
 #undef LSA_TILES
-    experts_combine_kernel<<<n, 256, 0, stream>>>(y, weights, out, top, width, chosen, experts,
+    experts_combine_kernel<4><<<dim3(n, (width + 1023) / 1024), 256, 0, stream>>>(y, weights, out, top, width, chosen, experts,
                                                  BesideExperts<bf16_t>{identity ? xb : nullptr, shared_gate, (const bf16_t*)shared_y, nullptr, nullptr, 0});
     LSA_LAUNCH_CHECK();
 }

@@ -184,8 +184,8 @@ LSA_EXPORT int lsa_gated_group_norm(int code, const float* y, const void* x, lon
     const int part = width / groups;
 #define LSA_LAUNCH(T, COLS) gated_group_norm_kernel<T, COLS><<<dim3(n_tokens, groups), 256, 0, stream>>>(y, (const T*)x, x_stride, skip, (const T*)gate, \
         gate_stride, weight, eps, (T*)out, part, value_dim, width)
-#define LSA_BY_COLS(T) do { if (part <= 256) LSA_LAUNCH(T, 1); else if (part <= 1024) LSA_LAUNCH(T, 4); else if (part <= 4096) LSA_LAUNCH(T, 16); \
-        else LSA_LAUNCH(T, 0); } while (0)
+#define LSA_BY_COLS(T) do { if (part <= 256) LSA_LAUNCH(T, 1); else if (part <= 512) LSA_LAUNCH(T, 2); else if (part <= 1024) LSA_LAUNCH(T, 4); else if (part <= 2048) LSA_LAUNCH(T, 8); \
+        else if (part <= 4096) LSA_LAUNCH(T, 16); else LSA_LAUNCH(T, 0); } while (0)
     if (code) LSA_BY_COLS(bf16_t); else LSA_BY_COLS(float);
 #undef LSA_BY_COLS
 #undef LSA_LAUNCH

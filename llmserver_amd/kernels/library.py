@@ -58,7 +58,7 @@ _SIGNATURES = {
     "lsa_latent_prepare": [c_int, _P, c_long, _P, _P, _P, c_float, _P, c_int, _P, _P, _P, c_int, _P, _P, c_int, _P, c_int, c_int, c_int,
                            c_int, c_int, c_int, c_int, c_int, _P],
     "lsa_gate_heads": [c_int, _P, _P, _P, c_int, c_int, _P, c_long, c_int, _P, c_int, c_int, c_int, c_int, _P],
-    "lsa_route_logits": [_P, _P, _P, c_int, c_int, c_int, _P],
+    "lsa_route_logits": [c_int, _P, _P, _P, c_int, c_int, c_int, _P],
     "lsa_route_top": [_P, c_int, c_int, _P, _P, c_int, c_int, c_int, c_int, _P, _P, c_float, c_int, _P, _P],
     "lsa_gated_pair_update": [_P, _P, c_int, c_int, _P, c_int, _P, _P, c_int, _P, _P, c_float, _P, c_int, c_int, c_int, _P],
     "lsa_differential_heads": [c_int, _P, c_float, c_float, c_float, _P, c_int, c_int, c_int, c_int, c_int, _P],

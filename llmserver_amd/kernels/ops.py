@@ -1044,13 +1044,12 @@ class HipOps(KernelNamespace):
             _check(gate_out, "gate_out", torch.float32, (n,))
         if not 1 <= top <= experts or experts > 3072:
             raise ValueError(f"the router kernel chooses 1 to {min(experts, 3072)} of up to 3072 experts, asked for {top} of {experts}")
-        wide = x if x.dtype == torch.float32 else x.float()
         if n <= self.LATENT_FEW_ROWS:          # few tokens: a kernel of a few microseconds instead of a library call
             logits = torch.empty((n, outputs), device=x.device, dtype=torch.float32)
-            _launched(self._part_library("experts").lsa_route_logits(_ptr(wide), _ptr(router), _ptr(logits), n, outputs, width, _stream()),
+            _launched(self._part_library("experts").lsa_route_logits(_code(x), _ptr(x), _ptr(router), _ptr(logits), n, outputs, width, _stream()),
                       "route_logits")
         else:
-            logits = torch.mm(wide, router.t())
+            logits = torch.mm(x if x.dtype == torch.float32 else x.float(), router.t())
         if scoring not in self.SCORINGS or (groups is not None and scoring != "sigmoid"):
             raise ValueError(f"the router kernel scores by {self.SCORINGS} (groups with sigmoid only), asked for {scoring!r}, groups {groups}")
         if (correction is not None or weight_scale != 1.0) and scoring != "softmax_all":

@@ -463,7 +463,7 @@ class TorchOps(KernelNamespace):
             assert wide.shape[0] == len(row_start)
             for t in range(wide.shape[0]):
                 slot = int(state_slots[int(token_row[t])])
-                old = state[slot, offset:offset + kept * channels].view(kept, channels)
+                old = state[slot, offset:offset + kept * channels].view(kept, channels) * (1.0 if int(positions[t]) else 0.0)
                 state[slot, offset:offset + kept * channels] = torch.cat([old[1:], wide[t:t + 1]], dim=0).reshape(-1)
 
     def gated_group_norm(self, y, x, skip, gate, weight, eps, out, heads, groups):
@@ -807,3 +807,56 @@ class ChunkedMemoryOps(TorchOps):
             state[slot, :matrix_size] = both[..., :value_dim].reshape(-1)
             state[slot, matrix_size:matrix_size + normaliser_size] = both[..., value_dim].reshape(-1)
             state[slot, matrix_size + normaliser_size:matrix_size + normaliser_size + heads] = top
+
+
+class ChunkedDecayOps(TorchOps):
+    """The twins, with the recurrences of one decay per head in their chunked form where a step brings ``chunked_from``
+    tokens more than it has rows: a row's tokens in chunks of ``chunk`` from its first token of the step; with ``L_t`` the
+    sum of ``log_keep`` from the chunk's first token to ``t``, the read-outs are ``(Q K^T * W) V + e^(L_t) q_t S_0`` with
+    ``W[t, j] = e^(L_t - L_j) take_j`` for ``j <= t``, and the state behind the chunk is
+    ``e^(L_last) S_0 + sum_j e^(L_last - L_j) take_j k_j v_j^T``."""
+
+    def __init__(self, chunk=64, chunked_from=64):
+        super().__init__()
+        self.chunk, self.chunked_from, self.chunked_steps = int(chunk), int(chunked_from), 0
+
+    def matrix_memory_chunks(self, n_tokens, rows):
+        return n_tokens // self.chunk + rows if n_tokens - rows >= self.chunked_from else 0
+
+    def decayed_recurrence(self, q, k, v, log_keep, take, q_scale, state, state_slots, row_start, row_len, row_ctx, out, heads, key_heads,
+                           dim, value_dim, sums=None, totals=None):
+        if sums is None:
+            assert totals is None
+            return super().decayed_recurrence(q, k, v, log_keep, take, q_scale, state, state_slots, row_start, row_len, row_ctx, out, heads,
+                                              key_heads, dim, value_dim)
+        n, size, each = out.shape[0], heads * dim * value_dim, heads // key_heads
+        assert tuple(sums.shape[1:]) == (heads, dim, value_dim) and sums.shape[0] >= n // self.chunk + len(row_len)
+        assert tuple(totals.shape) == (sums.shape[0], heads)
+        self.chunked_steps += 1
+        logs = log_keep.expand(n, heads)
+        steps = torch.ones(n, heads) if take is None else take
+        for row in range(len(row_len)):
+            start, count, end = int(row_start[row]), int(row_len[row]), int(row_ctx[row])
+            if count <= 0:
+                continue
+            slot = int(state_slots[row])
+            matrix = state[slot, :size].view(heads, dim, value_dim).clone()
+            if end - count == 0:
+                matrix.zero_()
+            for first in range(start, start + count, self.chunk):
+                tokens = slice(first, min(first + self.chunk, start + count))
+                m = tokens.stop - tokens.start
+                L = torch.cumsum(logs[tokens].double(), dim=0)                                       # [m, h]
+                queries = q[tokens].float().view(m, key_heads, dim).repeat_interleave(each, dim=1) * q_scale
+                keys = k[tokens].float().view(m, key_heads, dim).repeat_interleave(each, dim=1)
+                values = v[tokens].float().reshape(m, heads, value_dim)
+                behind = torch.tril(torch.ones(m, m, dtype=torch.bool))[:, :, None]                   # j <= t
+                apart = torch.where(behind, L[:, None, :] - L[None, :, :], torch.tensor(-float("inf"), dtype=torch.float64))
+                weights = torch.exp(apart.float()) * steps[tokens][None, :, :]                        # [t, j, h]
+                scores = torch.einsum("thd,jhd->tjh", queries, keys) * weights
+                read = torch.einsum("tjh,jhv->thv", scores, values) \
+                    + torch.exp(L.float())[:, :, None] * torch.einsum("thd,hdv->thv", queries, matrix)
+                out[tokens] = read.reshape(m, -1)
+                to_last = torch.exp((L[-1][None, :] - L).float()) * steps[tokens]                      # [j, h]
+                matrix = torch.exp(L[-1].float())[:, None, None] * matrix + torch.einsum("jh,jhd,jhv->hdv", to_last, keys, values)
+            state[slot, :size] = matrix.reshape(-1)
