@@ -3,7 +3,7 @@
 Layers with the same cache needs form a group; every group has its own pages, its own allocator
 and, per request, its own block table.  A group that keeps all keys frees a request's pages when
 the request ends; a group with a window also frees a page as soon as every key on it has fallen
-out of the window of all queries still to come.  Freed pages are used again.  Beside the pages
+out of the window (or the chunk) of all queries still to come.  Freed pages are used again.  Beside the pages
 there are slots for per-request state of fixed size.
 
 Page layout (one cache, i.e. one layer): keys ``[pages, kv_heads, page_size, head_dim]``, values
@@ -69,9 +69,7 @@ class CacheGroup:
 
     def first_needed_block(self, num_computed: int) -> int:
         """First logical block a query at position >= num_computed can still see."""
-        if self.spec.window is None:
-            return 0
-        return max(0, num_computed - self.spec.window + 1) // self.page_size
+        return self.spec.first_key(num_computed) // self.page_size
 
 
 class RequestCache:
@@ -138,7 +136,7 @@ class CacheManager:
         self.state: Dict[int, torch.Tensor] = {}
         self.requests: Dict[object, RequestCache] = {}
         self.prefix_caching_possible = bool(self.groups) and not self.state_specs and all(
-            group.spec.window is None for group in self.groups)
+            not group.spec.bounded for group in self.groups)
         if allocate_storage:
             self._allocate_storage()
 
@@ -266,11 +264,11 @@ class CacheManager:
             raise
 
     def advance(self, request_id, num_computed: int) -> None:
-        """Tokens ``< num_computed`` are in the cache; give back pages a window has passed."""
+        """Tokens ``< num_computed`` are in the cache; give back pages that a window has passed or whose chunks have ended."""
         record = self.record(request_id)
         record.num_computed = num_computed
         for group in self.groups:
-            if group.spec.window is None:
+            if not group.spec.bounded:
                 continue
             table = record.tables[group.index]
             for block in range(min(group.first_needed_block(num_computed), len(table))):

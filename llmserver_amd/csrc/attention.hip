@@ -42,6 +42,12 @@ constexpr float NEG_INF = -__builtin_huge_valf();
 // Two wavefronts per SIMD while the double-buffered operands of a step fit into 256 registers.
 #define LSA_MIN_WAVES (LSA_ND <= 8 ? 2 : 1)
 
+#if LSA_BF16
+typedef bf16_t elem_t;
+#else
+typedef float elem_t;
+#endif
+
 struct Item { int row, q0, k_begin, k_end; };
 
 struct Geometry {
@@ -51,7 +57,22 @@ struct Geometry {
     const float* sinks;       // [n_q] or null: exp(sinks[head]) joins every softmax's denominator (no key, no value)
     float cap, cap_inverse;   // cap > 0: a scaled score s becomes cap * tanh(s / cap) before the mask
     float scale_inverse;      // 1 / scale (0 for a scale of 0), for the kernel that keeps its scores unscaled
+    int chunk;                // > 0: a query sees keys of its own chunk only, chunks of so many positions counted from 0
+    const float* slopes;      // [n_q] or null: a score, after scale and cap, loses slopes[head] times the positions between query and key
+    const elem_t* gates;      // [tokens][gate_stride] or null: a head's result is multiplied by sigmoid(gates[token][head])
+    long gate_stride;
 };
+
+// The first key that a query at `position` sees.
+__device__ __forceinline__ int first_key_of(int position, const Geometry& g) {
+    const int first = g.window > 0 ? position - g.window + 1 : 0;
+    return g.chunk > 0 ? max(first, position / g.chunk * g.chunk) : first;
+}
+
+// What a head's result is multiplied by at the very end, beside one over its softmax's sum.
+__device__ __forceinline__ float gate_of(const Geometry& g, size_t token, int head) {
+    return g.gates != nullptr ? 1.f / (1.f + expf(-(float)g.gates[token * g.gate_stride + head])) : 1.f;
+}
 
 __device__ __forceinline__ float tanh_of(float x) {
 #if LSA_BF16
@@ -95,11 +116,9 @@ struct DecodeFusion {
 };
 
 #if LSA_BF16
-typedef bf16_t elem_t;
 constexpr int KEY_STEP = 32;                 // keys per loop step (one 16x16x32 MFMA in the output product)
 constexpr int NS = (D + 31) / 32;            // 32-dim steps of the score product
 #else
-typedef float elem_t;
 constexpr int KEY_STEP = 16;
 constexpr int NS = D / 16;                   // 16-dim steps (four 16x16x4 MFMAs each)
 #endif
@@ -112,7 +131,8 @@ constexpr int NS = D / 16;                   // 16-dim steps (four 16x16x4 MFMAs
 // of two tiles (the plan says so), and the workgroup merges them itself through LDS and writes the output: no partial
 // results in memory, no merge launch.  For steps whose contexts are short, where that launch costs as much as the
 // attention, and for steps of many rows, whose tiles get no more ranges than that anyway.
-template <int MODE, bool PLAIN, int WG_RANGES>
+// BIAS: scores fall with the distance between query and key (Geometry::slopes); without it nothing of that is in the code.
+template <int MODE, bool PLAIN, int WG_RANGES, bool BIAS>
 __global__ __launch_bounds__(256, LSA_MIN_WAVES) void paged_attention_kernel(
     const elem_t* __restrict__ q, long q_token_stride, elem_t* __restrict__ out,
     const elem_t* keys, const elem_t* values,
@@ -192,6 +212,9 @@ __global__ __launch_bounds__(256, LSA_MIN_WAVES) void paged_attention_kernel(
     const bool pair_valid = pair_token < g.tokens_per_tile && item.q0 + pair_token < n && pair_head_in_group < g.group;
     const int q_pos = pair_valid ? first_pos + item.q0 + pair_token : -1;
     const int head = kv_head * g.group + pair_head_in_group;
+    const int first_seen = first_key_of(q_pos, g);
+    float slope = 0.f;
+    if constexpr (BIAS) slope = g.slopes[pair_valid ? head : kv_head * g.group];
     // Decode steps: the item that ends at the row's new token takes that token's key and value from the projection,
     // and walks the pages up to the key before it.
     const bool takes_new_token = NEW_TOKEN && item.k_begin < item.k_end && item.k_end == ctx;
@@ -465,8 +488,9 @@ __global__ __launch_bounds__(256, LSA_MIN_WAVES) void paged_attention_kernel(
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 const int kpos = kt + 16 * t2 + 4 * quad + r;
-                const bool seen = kpos >= k_begin && kpos < k_end && kpos <= q_pos && (g.window <= 0 || kpos > q_pos - g.window);
-                const float v = seen ? capped(s4[r] * g.scale, g) : NEG_INF;
+                const bool seen = kpos >= k_begin && kpos < k_end && kpos <= q_pos && kpos >= first_seen;
+                float v = seen ? capped(s4[r] * g.scale, g) : NEG_INF;
+                if constexpr (BIAS) v -= slope * (float)(q_pos - kpos);
                 sv[4 * t2 + r] = v;
                 tile_max = fmaxf(tile_max, v);
             }
@@ -484,8 +508,9 @@ __global__ __launch_bounds__(256, LSA_MIN_WAVES) void paged_attention_kernel(
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 const int kpos = kt + 4 * quad + r;
-                const bool seen = kpos >= k_begin && kpos < k_end && kpos <= q_pos && (g.window <= 0 || kpos > q_pos - g.window);
-                const float v = seen ? capped(s4[r] * g.scale, g) : NEG_INF;
+                const bool seen = kpos >= k_begin && kpos < k_end && kpos <= q_pos && kpos >= first_seen;
+                float v = seen ? capped(s4[r] * g.scale, g) : NEG_INF;
+                if constexpr (BIAS) v -= slope * (float)(q_pos - kpos);
                 sv[r] = v;
                 tile_max = fmaxf(tile_max, v);
             }
@@ -603,7 +628,7 @@ __global__ __launch_bounds__(256, LSA_MIN_WAVES) void paged_attention_kernel(
             weight[w] = m == NEG_INF ? 0.f : expf(m - top);
             total += weight[w] * ranges_sum[first_wave + w][col];
         }
-        const float inv = inverse_of_sum(total, top, g.sinks, head);
+        const float inv = inverse_of_sum(total, top, g.sinks, head) * gate_of(g, token0 + pair_token, head);
         elem_t* o = out + ((size_t)(token0 + pair_token) * g.n_q + head) * D + 4 * quad;
 #pragma unroll
         for (int c = 0; c < ND; ++c) {
@@ -623,7 +648,7 @@ __global__ __launch_bounds__(256, LSA_MIN_WAVES) void paged_attention_kernel(
     }
     if (!pair_valid) return;
     if (slot < 0) {
-        const float inv = inverse_of_sum(run_sum, run_max, g.sinks, head);
+        const float inv = inverse_of_sum(run_sum, run_max, g.sinks, head) * gate_of(g, token0 + pair_token, head);
         elem_t* o = out + ((size_t)(token0 + pair_token) * g.n_q + head) * D + 4 * quad;
 #pragma unroll
         for (int c = 0; c < ND; ++c) {
@@ -745,7 +770,7 @@ __device__ __forceinline__ void loads_landed_then_barrier() {
 // combines a tile's slots.  first < 0 (or no `tile_slots` at all): the entry holds all keys and writes the output.
 struct TileSlots { int first, stride; };
 
-template <int SUB, int HALVES>
+template <int SUB, int HALVES, bool BIAS>
 __global__ __launch_bounds__(256 * HALVES, LSA_TILE_MIN_WAVES(SUB)) void paged_attention_tile_kernel(
     const elem_t* __restrict__ q, long q_token_stride, elem_t* __restrict__ out,
     const elem_t* __restrict__ keys, const elem_t* __restrict__ values,
@@ -772,13 +797,17 @@ __global__ __launch_bounds__(256 * HALVES, LSA_TILE_MIN_WAVES(SUB)) void paged_a
     const int pair_token = col / g.gheads, pair_head_in_group = gtile * g.gheads + col % g.gheads;
     const int head = kv_head * g.group + pair_head_in_group;
     bool pair_valid[SUB];
-    int q_pos[SUB];
+    int q_pos[SUB], first_seen[SUB];
 #pragma unroll
     for (int u = 0; u < SUB; ++u) {
         const int token = q0 + u * g.tokens_per_tile + pair_token;
         pair_valid[u] = pair_token < g.tokens_per_tile && token < n && pair_head_in_group < g.group;
         q_pos[u] = pair_valid[u] ? first_pos + token : -1;
+        first_seen[u] = first_key_of(q_pos[u], g);
     }
+    // (scores stay in units of 1 / scale here, and so does what they lose per position)
+    float slope = 0.f;
+    if constexpr (BIAS) slope = g.slopes[min(head, g.n_q - 1)] * g.scale_inverse;
     const int* row_table = table + (size_t)row * table_stride;
     const int ps = g.page_size;
     const size_t kv_head_keys = (size_t)kv_head * ps * D, kv_head_values = (size_t)kv_head * D * ps;
@@ -786,7 +815,7 @@ __global__ __launch_bounds__(256 * HALVES, LSA_TILE_MIN_WAVES(SUB)) void paged_a
     // Keys this wavefront's pairs can see at all: [wave_lo, wave_hi).
     const int wave_tokens = max(0, min(SUB * g.tokens_per_tile, n - q0));
     const int wave_hi = wave_tokens > 0 ? first_pos + q0 + wave_tokens : 0;
-    const int wave_lo = g.window > 0 ? max(0, first_pos + q0 - g.window + 1) : 0;
+    const int wave_lo = max(0, first_key_of(first_pos + q0, g));
     const int q_pos_min = first_pos + q0;                       // smallest position among the wavefront's valid pairs
     const float scale_log2 = g.scale * 1.44269504088896340736f;
 
@@ -903,7 +932,7 @@ __global__ __launch_bounds__(256 * HALVES, LSA_TILE_MIN_WAVES(SUB)) void paged_a
     // The steps that every pair of the wavefront sees completely (they need no mask) lie in [full_from, full_to]; the
     // steps that have anything for its pairs in (active_from, active_to).
     const bool whole_tiles = wave_tokens == SUB * g.tokens_per_tile && g.gheads * g.tokens_per_tile == 16 && (gtile + 1) * g.gheads <= g.group;
-    const int full_from = !whole_tiles ? 0x7fffffff : g.window > 0 ? max(k_begin, first_pos + q0 + wave_tokens - g.window) : k_begin;
+    const int full_from = !whole_tiles ? 0x7fffffff : max(k_begin, first_key_of(first_pos + q0 + wave_tokens - 1, g));
     const int full_to = min(k_end - 32, q_pos_min - 31);
     // Scores stay as the products left them; the scale (in units of ln 2, so that the exponential is one
     // instruction) goes into the multiply-add that also subtracts the running maximum.  FULL: every key of
@@ -927,15 +956,21 @@ __global__ __launch_bounds__(256 * HALVES, LSA_TILE_MIN_WAVES(SUB)) void paged_a
 #pragma unroll
                 for (int u = 0; u < SUB; ++u) s4[u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[u][s], s4[u], 0, 0, 0);
             }
+            float nearest[SUB];
+            if constexpr (BIAS) {
+#pragma unroll
+                for (int u = 0; u < SUB; ++u) nearest[u] = -slope * (float)(q_pos[u] - (kt + 8 * quad + 4 * t2));      // what the first of the four loses
+            }
 #pragma unroll
             for (int u = 0; u < SUB; ++u)
 #pragma unroll
                 for (int r = 0; r < 4; ++r) {
                     float v = s4[u][r];
                     if (g.cap > 0.f) v = capped(v * g.scale, g) * g.scale_inverse;       // (scores stay in units of 1 / scale here)
+                    if constexpr (BIAS) v += __builtin_fmaf(slope, (float)r, nearest[u]);
                     if (!FULL) {
                         const int kpos = kt + 8 * quad + 4 * t2 + r;
-                        const bool seen = kpos >= k_begin && kpos < k_end && kpos <= q_pos[u] && (g.window <= 0 || kpos > q_pos[u] - g.window);
+                        const bool seen = kpos >= k_begin && kpos < k_end && kpos <= q_pos[u] && kpos >= first_seen[u];
                         v = seen ? v : NEG_INF;
                     }
                     sv[u][4 * t2 + r] = v;
@@ -1078,8 +1113,9 @@ __global__ __launch_bounds__(256 * HALVES, LSA_TILE_MIN_WAVES(SUB)) void paged_a
                 }
                 continue;
             }
-            const float inv = inverse_of_sum(total, top == NEG_INF ? NEG_INF : top * g.scale, g.sinks, head);
-            elem_t* o = out + ((size_t)(row_start[row] + q0 + u * g.tokens_per_tile + pair_token) * g.n_q + head) * D + 4 * quad;
+            const size_t token = (size_t)(row_start[row] + q0 + u * g.tokens_per_tile + pair_token);
+            const float inv = inverse_of_sum(total, top == NEG_INF ? NEG_INF : top * g.scale, g.sinks, head) * gate_of(g, token, head);
+            elem_t* o = out + (token * g.n_q + head) * D + 4 * quad;
 #pragma unroll
             for (int c = 0; c < ND; ++c) {
                 const f32x4 other = *reinterpret_cast<const f32x4*>(block + (c * 64 + lane) * 4);
@@ -1110,8 +1146,9 @@ __global__ __launch_bounds__(256 * HALVES, LSA_TILE_MIN_WAVES(SUB)) void paged_a
             }
             continue;
         }
-        const float inv = inverse_of_sum(total, run_max[u] == NEG_INF ? NEG_INF : run_max[u] * g.scale, g.sinks, head);
-        elem_t* o = out + ((size_t)(row_start[row] + q0 + u * g.tokens_per_tile + pair_token) * g.n_q + head) * D + 4 * quad;
+        const size_t token = (size_t)(row_start[row] + q0 + u * g.tokens_per_tile + pair_token);
+        const float inv = inverse_of_sum(total, run_max[u] == NEG_INF ? NEG_INF : run_max[u] * g.scale, g.sinks, head) * gate_of(g, token, head);
+        elem_t* o = out + (token * g.n_q + head) * D + 4 * quad;
 #pragma unroll
         for (int c = 0; c < ND; ++c) {
             bf16x4 r4;
@@ -1160,7 +1197,9 @@ __global__ __launch_bounds__(256) void paged_attention_tile_kernel_f32(
     const size_t page_elems = (size_t)g.n_kv * ps * D;
     const int wave_tokens = max(0, min(g.tokens_per_tile, n - q0));
     const int wave_hi = wave_tokens > 0 ? first_pos + q0 + wave_tokens : 0;                  // keys this wavefront's pairs can see: [wave_lo, wave_hi)
-    const int wave_lo = g.window > 0 ? max(0, first_pos + q0 - g.window + 1) : 0;
+    const int wave_lo = max(0, first_key_of(first_pos + q0, g));
+    const int first_seen = first_key_of(q_pos, g);
+    const float slope = g.slopes != nullptr ? g.slopes[min(head, g.n_q - 1)] : 0.f;
 
     f32x4 qf[NS];
 #pragma unroll
@@ -1248,8 +1287,8 @@ __global__ __launch_bounds__(256) void paged_attention_tile_kernel_f32(
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
             const int kpos = kt + 4 * quad + r;
-            const bool seen = kpos >= k_begin && kpos < k_end && kpos <= q_pos && (g.window <= 0 || kpos > q_pos - g.window);
-            sv[r] = seen ? capped(s4[r] * g.scale, g) : NEG_INF;
+            const bool seen = kpos >= k_begin && kpos < k_end && kpos <= q_pos && kpos >= first_seen;
+            sv[r] = seen ? capped(s4[r] * g.scale, g) - slope * (float)(q_pos - kpos) : NEG_INF;
             step_max = fmaxf(step_max, sv[r]);
         }
         step_max = fmaxf(step_max, __shfl_xor(step_max, 16, 64));
@@ -1296,8 +1335,9 @@ __global__ __launch_bounds__(256) void paged_attention_tile_kernel_f32(
     run_sum += __shfl_xor(run_sum, 16, 64);
     run_sum += __shfl_xor(run_sum, 32, 64);
     if (!pair_valid) return;
-    const float inv = inverse_of_sum(run_sum, run_max, g.sinks, head);
-    float* o = out + ((size_t)(row_start[row] + q0 + pair_token) * g.n_q + head) * D + 4 * quad;
+    const size_t token = (size_t)(row_start[row] + q0 + pair_token);
+    const float inv = inverse_of_sum(run_sum, run_max, g.sinks, head) * gate_of(g, token, head);
+    float* o = out + (token * g.n_q + head) * D + 4 * quad;
 #pragma unroll
     for (int c = 0; c < ND; ++c) *reinterpret_cast<f32x4*>(o + 16 * c) = acc[c] * inv;
 }
@@ -1351,7 +1391,10 @@ __global__ __launch_bounds__(MERGE_WAVES * 64) void merge_kernel(
             weighted += w * sum[i];
         }
         const float total = wave_sum(weighted);
-        if (lane == 0) inv_total = inverse_of_sum(total, top, g.sinks, kv_head * g.group + pair_head_in_group);
+        if (lane == 0) {
+            const int head = kv_head * g.group + pair_head_in_group;
+            inv_total = inverse_of_sum(total, top, g.sinks, head) * gate_of(g, (size_t)(row_start[m.row] + m.q0 + pair_token), head);
+        }
     }
     // The partial results do not depend on the weights: their first loads are issued before the barrier.
     const float* acc = part_acc + base * D;
@@ -1423,9 +1466,11 @@ LSA_EXPORT int lsa_paged_attention(
     float scale,
     int window, int page_size, int n_q, int n_kv, int gheads, int tokens_per_tile, int gtiles,
     int decode_fusion, const float* q_weight, const float* k_weight, float norm_eps, const float* cos_sin, int tiles_per_workgroup,
-    int merge_in_workgroup, int tile_halves, const float* sinks, float softcap, hipStream_t stream) {
+    int merge_in_workgroup, int tile_halves, const float* sinks, float softcap, int chunk, const float* slopes, const void* gates, long gate_stride,
+    hipStream_t stream) {
     if (n_items <= 0 && n_tiles <= 0) return 0;
-    if (softcap < 0.f) return -1;
+    if (softcap < 0.f || chunk < 0 || (gates != nullptr && gate_stride < n_q)) return -1;
+    if (slopes != nullptr && (decode_fusion || !(scale > 0.f))) return -1;      // (the fused start takes scores without a bias only)
     // decode_fusion (see DecodeFusion::mode): the caller promises that every row of the step brings one token.
     DecodeFusion fusion = {q_weight, k_weight, cos_sin, norm_eps, decode_fusion};
     if (decode_fusion != 0 && decode_fusion != 1 && decode_fusion != 3) return -1;
@@ -1434,6 +1479,7 @@ LSA_EXPORT int lsa_paged_attention(
     g.n_q = n_q; g.n_kv = n_kv; g.group = n_q / n_kv; g.gheads = gheads; g.tokens_per_tile = tokens_per_tile;
     g.gtiles = gtiles; g.page_size = page_size; g.window = window; g.scale = scale; g.sinks = sinks;
     g.cap = softcap; g.cap_inverse = softcap > 0.f ? 1.f / softcap : 0.f; g.scale_inverse = scale != 0.f ? 1.f / scale : 0.f;
+    g.chunk = chunk; g.slopes = slopes; g.gates = (const elem_t*)gates; g.gate_stride = gate_stride;
     g.page_magic = (unsigned)(((1ull << 32) + page_size - 1) / page_size);
     if (n_tiles > 0) {
 #if LSA_BF16
@@ -1442,7 +1488,8 @@ LSA_EXPORT int lsa_paged_attention(
         if (page_size % 8 != 0) return -1;
         dim3 tgrid(n_tiles * n_kv * gtiles);
         if (tile_halves != 1 && tile_halves != MAX_HALVES) return -1;
-#define LSA_LAUNCH_TILES(SUB, HALVES) paged_attention_tile_kernel<SUB, HALVES><<<tgrid, 256 * HALVES, 0, stream>>>( \
+#define LSA_LAUNCH_TILES(SUB, HALVES) do { if (slopes != nullptr) LSA_LAUNCH_TILES_OF(SUB, HALVES, true); else LSA_LAUNCH_TILES_OF(SUB, HALVES, false); } while (0)
+#define LSA_LAUNCH_TILES_OF(SUB, HALVES, BIAS) paged_attention_tile_kernel<SUB, HALVES, BIAS><<<tgrid, 256 * HALVES, 0, stream>>>( \
                 (const elem_t*)q, q_token_stride, (elem_t*)out, (const elem_t*)keys, (const elem_t*)values, table, table_stride, \
                 row_start, row_len, row_ctx, (const Item*)tiles, (const TileSlots*)tile_slots, part_acc, part_ml, g)
         if (tile_slots != nullptr && (part_acc == nullptr || part_ml == nullptr || n_merges <= 0)) return -1;
@@ -1451,6 +1498,7 @@ LSA_EXPORT int lsa_paged_attention(
         else if (tile_halves == 1) LSA_LAUNCH_TILES(MAX_SUB, 1);
         else LSA_LAUNCH_TILES(MAX_SUB, MAX_HALVES);
 #undef LSA_LAUNCH_TILES
+#undef LSA_LAUNCH_TILES_OF
         const int terr = (int)hipGetLastError();
         if (terr) return terr;
 #else
@@ -1469,30 +1517,37 @@ LSA_EXPORT int lsa_paged_attention(
         if (merge_in_workgroup && ((merge_in_workgroup != 2 && merge_in_workgroup != 4) || n_items % 4 != 0 || n_merges != 0)) return -1;
         dim3 grid((n_items + 3) / 4, n_kv * gtiles);
 #define LSA_LAUNCH_ITEMS(MODE, PLAIN) LSA_LAUNCH_ITEMS_MERGE(MODE, PLAIN, 0)
-#define LSA_LAUNCH_ITEMS_MERGE(MODE, PLAIN, RANGES) paged_attention_kernel<MODE, PLAIN, RANGES><<<grid, 256, 0, stream>>>( \
+#define LSA_LAUNCH_ITEMS_MERGE(MODE, PLAIN, RANGES) LSA_LAUNCH_ITEMS_OF(MODE, PLAIN, RANGES, false)
+#define LSA_LAUNCH_ITEMS_OF(MODE, PLAIN, RANGES, BIAS) paged_attention_kernel<MODE, PLAIN, RANGES, BIAS><<<grid, 256, 0, stream>>>( \
             (const elem_t*)q, q_token_stride, (elem_t*)out, (const elem_t*)keys, (const elem_t*)values, table, table_stride, \
             row_start, row_len, row_ctx, (const Item*)items, item_slot, n_items, part_acc, part_ml, g, fusion)
+        if (slopes != nullptr) {
+            if (merge_in_workgroup == 4) LSA_LAUNCH_ITEMS_OF(0, false, 4, true);
+            else if (merge_in_workgroup == 2) LSA_LAUNCH_ITEMS_OF(0, false, 2, true);
+            else LSA_LAUNCH_ITEMS_OF(0, false, 0, true);
+        } else {
 #if LSA_BF16
-        const bool plain = q_weight != nullptr && cos_sin != nullptr;
-        if (merge_in_workgroup && decode_fusion && !plain) return -1;      // the caller asks lsa_attention_merges_in_workgroup first
-        if (merge_in_workgroup == 4 && decode_fusion == 3) LSA_LAUNCH_ITEMS_MERGE(3, true, 4);
-        else if (merge_in_workgroup == 4 && decode_fusion == 1) LSA_LAUNCH_ITEMS_MERGE(1, true, 4);
-        else if (merge_in_workgroup == 4) LSA_LAUNCH_ITEMS_MERGE(0, false, 4);
-        else if (merge_in_workgroup == 2 && decode_fusion == 3) LSA_LAUNCH_ITEMS_MERGE(3, true, 2);
-        else if (merge_in_workgroup == 2 && decode_fusion == 1) LSA_LAUNCH_ITEMS_MERGE(1, true, 2);
-        else if (merge_in_workgroup == 2) LSA_LAUNCH_ITEMS_MERGE(0, false, 2);
-        else if (decode_fusion == 3 && plain) LSA_LAUNCH_ITEMS(3, true);
-        else if (decode_fusion == 3) LSA_LAUNCH_ITEMS(3, false);
-        else if (decode_fusion == 1 && plain) LSA_LAUNCH_ITEMS(1, true);
-        else if (decode_fusion == 1) LSA_LAUNCH_ITEMS(1, false);
-        else
+            const bool plain = q_weight != nullptr && cos_sin != nullptr;
+            if (merge_in_workgroup && decode_fusion && !plain) return -1;      // the caller asks lsa_attention_merges_in_workgroup first
+            if (merge_in_workgroup == 4 && decode_fusion == 3) LSA_LAUNCH_ITEMS_MERGE(3, true, 4);
+            else if (merge_in_workgroup == 4 && decode_fusion == 1) LSA_LAUNCH_ITEMS_MERGE(1, true, 4);
+            else if (merge_in_workgroup == 4) LSA_LAUNCH_ITEMS_MERGE(0, false, 4);
+            else if (merge_in_workgroup == 2 && decode_fusion == 3) LSA_LAUNCH_ITEMS_MERGE(3, true, 2);
+            else if (merge_in_workgroup == 2 && decode_fusion == 1) LSA_LAUNCH_ITEMS_MERGE(1, true, 2);
+            else if (merge_in_workgroup == 2) LSA_LAUNCH_ITEMS_MERGE(0, false, 2);
+            else if (decode_fusion == 3 && plain) LSA_LAUNCH_ITEMS(3, true);
+            else if (decode_fusion == 3) LSA_LAUNCH_ITEMS(3, false);
+            else if (decode_fusion == 1 && plain) LSA_LAUNCH_ITEMS(1, true);
+            else if (decode_fusion == 1) LSA_LAUNCH_ITEMS(1, false);
+            else LSA_LAUNCH_ITEMS(0, false);
 #else
-        if (merge_in_workgroup == 4) LSA_LAUNCH_ITEMS_MERGE(0, false, 4);
-        else if (merge_in_workgroup == 2) LSA_LAUNCH_ITEMS_MERGE(0, false, 2);
-        else
+            if (merge_in_workgroup == 4) LSA_LAUNCH_ITEMS_MERGE(0, false, 4);
+            else if (merge_in_workgroup == 2) LSA_LAUNCH_ITEMS_MERGE(0, false, 2);
+            else LSA_LAUNCH_ITEMS(0, false);
 #endif
-        LSA_LAUNCH_ITEMS(0, false);
+        }
 #undef LSA_LAUNCH_ITEMS_MERGE
+#undef LSA_LAUNCH_ITEMS_OF
 #undef LSA_LAUNCH_ITEMS
         err = (int)hipGetLastError();
     }

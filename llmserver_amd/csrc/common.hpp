@@ -59,6 +59,59 @@ __device__ inline float block_sum(float v, float* scratch) {
     return total;
 }
 
+// Puts 64 consecutive tokens of one KV head, staged in LDS as [VT_TOKENS][pitch] with `filled` numbers a token, into their
+// pages values[page][kv_head][:][slot], zeros for the dimensions from `filled` to d.  Four slots of one dimension go out at
+// a time (8 or 16 bytes) where four tokens are neighbours in one page, which is the rule inside a portion; a page's
+// [d][page_size] block is contiguous, so these stores coalesce.  256 threads; whoever wrote the tile need not have waited.
+constexpr int VT_TOKENS = 64;
+template <typename T>
+__device__ __forceinline__ void store_value_tile(const T* tile, int pitch, int token0, int kv_head, int filled, T* __restrict__ values,
+                                                 const int* __restrict__ table, int table_stride, const int* __restrict__ token_row,
+                                                 const int* __restrict__ positions, int page_size, int n_kv, int d, int n_tokens) {
+    __shared__ long group_base[VT_TOKENS / 4];             // element offset of the group's first slot in `values`, or -1
+    __shared__ unsigned char covered[VT_TOKENS];           // token goes out with its group
+    // Four tokens go out together if they are one request's neighbours starting at a position that is a multiple
+    // of four; the groups are laid so that this holds when the tile lies inside one portion.
+    const int shift = (4 - (positions[min(token0, n_tokens - 1)] & 3)) & 3;
+    if (threadIdx.x < VT_TOKENS) covered[threadIdx.x] = 0;
+    __syncthreads();
+    if (threadIdx.x < VT_TOKENS / 4) {
+        const int local = shift + 4 * threadIdx.x, first = token0 + local;
+        long base = -1;
+        if (local + 3 < VT_TOKENS && first + 3 < n_tokens) {
+            const int row = token_row[first], pos = positions[first];
+            bool together = (pos & 3) == 0;
+            for (int r = 1; r < 4; ++r) together = together && token_row[first + r] == row && positions[first + r] == pos + r;
+            const int p = table[(size_t)row * table_stride + pos / page_size];
+            if (together && p >= 0) {
+                base = (((long)p * n_kv + kv_head) * d) * page_size + pos % page_size;
+                for (int r = 0; r < 4; ++r) covered[local + r] = 1;
+            }
+        }
+        group_base[threadIdx.x] = base;
+    }
+    __syncthreads();
+    for (int e = threadIdx.x; e < (VT_TOKENS / 4) * d; e += 256) {
+        const int g = e & (VT_TOKENS / 4 - 1), i = e / (VT_TOKENS / 4);      // neighbouring threads: neighbouring groups of slots
+        const long base = group_base[g];
+        if (base < 0) continue;
+        T four[4];
+#pragma unroll
+        for (int r = 0; r < 4; ++r) four[r] = i < filled ? tile[(shift + 4 * g + r) * pitch + i] : (T)0.f;
+        T* dst = values + base + (size_t)i * page_size;
+        if (sizeof(T) == 2) *reinterpret_cast<uint2*>(dst) = *reinterpret_cast<const uint2*>(four);
+        else *reinterpret_cast<uint4*>(dst) = *reinterpret_cast<const uint4*>(four);
+    }
+    for (int e = threadIdx.x; e < VT_TOKENS * d; e += 256) {                  // the tokens that are in no such group
+        const int t = e & (VT_TOKENS - 1), i = e / VT_TOKENS;
+        const int token = token0 + t;
+        if (covered[t] || token >= n_tokens) continue;
+        const int pos = positions[token];
+        const int p = table[(size_t)token_row[token] * table_stride + pos / page_size];
+        if (p >= 0) values[(((size_t)p * n_kv + kv_head) * d + i) * page_size + pos % page_size] = i < filled ? tile[t * pitch + i] : (T)0.f;
+    }
+}
+
 }  // namespace lsa
 
 #define LSA_EXPORT extern "C" __attribute__((visibility("default")))

@@ -4,8 +4,10 @@
 // a token's output row is the weighted sum over its pairs of the expert's down rows against the pair's hidden row.
 // Sums are 32-bit; the hidden row is rounded once to the activations' type; the output is float32.
 //
+// Experts without a gate (`plain`) have one matrix that reads the token, and max(up, 0)^2 in place of silu(gate) * up.
+//
 // Beside the experts that have matrices there may be identity experts: choices from `experts` on, whose output is the token's
-// row itself.  And there may be a shared expert that every token uses, weighted by a gate of one number a token: its
+// row itself.  And there may be a shared expert that every token uses, possibly weighted by a gate of one number a token: its
 // products are made inside the same two kernels (steps of few tokens), or its output comes ready made.
 #include "common.hpp"
 
@@ -22,6 +24,11 @@ __device__ __forceinline__ float gated_activation(float g, float u, float limit)
         return g / (1.f + expf(-1.702f * g)) * (u + 1.f);
     }
     return g / (1.f + expf(-g)) * u;
+}
+
+__device__ __forceinline__ float rectified_square(float u) {
+    u = fmaxf(u, 0.f);
+    return u * u;
 }
 
 // Dot product of a weight row with a vector in LDS, a wavefront wide: 16-byte pieces where the length allows.
@@ -207,7 +214,7 @@ __global__ __launch_bounds__(256) void experts_gate_up_kernel(const T* __restric
                                                               const int* __restrict__ chosen, T* __restrict__ hidden, int top,
                                                               int inter, int width, int experts, int columns_per_block, bool in_lds,
                                                               float limit, int identity, const T* __restrict__ shared_gate_up,
-                                                              T* __restrict__ shared_hidden, int shared_inter) {
+                                                              T* __restrict__ shared_hidden, int shared_inter, int plain) {
     extern __shared__ __align__(16) unsigned char lds_bytes[];
     const int slots = top + (shared_gate_up ? 1 : 0), t = blockIdx.x / slots, slot = blockIdx.x - t * slots;
     const bool shared = slot == top;
@@ -224,10 +231,20 @@ __global__ __launch_bounds__(256) void experts_gate_up_kernel(const T* __restric
         x_lds = staged;
     }
     expert = expert < 0 ? 0 : expert >= experts ? experts - 1 : expert;
-    const T* base = shared ? shared_gate_up : gate_up + (size_t)expert * 2 * inter * width;
+    const T* base = shared ? shared_gate_up : gate_up + (size_t)expert * (plain ? 1 : 2) * inter * width;
     T* result = shared ? shared_hidden + (size_t)t * shared_inter : hidden + (size_t)pair * inter;
     if (shared) inter = shared_inter;
     const int f0 = blockIdx.y * columns_per_block, f1 = min(inter, f0 + columns_per_block);
+    if (plain) {                                             // two columns at once, so that as many loads are in flight
+        for (int f = f0 + wave; f < f1; f += 2 * waves) {
+            const int other = min(f + waves, f1 - 1);
+            float a, b;
+            wave_dot2(base + (size_t)f * width, base + (size_t)other * width, x_lds, width, lane, a, b);
+            if (lane == 0) result[f] = (T)rectified_square(a);
+            if (lane == 0 && f + waves < f1) result[f + waves] = (T)rectified_square(b);
+        }
+        return;
+    }
     for (int f = f0 + wave; f < f1; f += waves) {
         float g, u;
         wave_dot2(base + (size_t)f * width, base + (size_t)(inter + f) * width, x_lds, width, lane, g, u);
@@ -242,9 +259,9 @@ __global__ __launch_bounds__(256) void experts_gate_up_kernel(const T* __restric
 // token's gate: shared_y ready made, or shared_down[c] . shared_hidden[t].
 template <typename T> struct BesideExperts {
     const T* x;                     // [tokens][width], or nullptr: no identity experts
-    const float* gate;              // [tokens]: what the shared expert's output is multiplied by, or nullptr: no shared expert
+    const float* gate;              // [tokens]: what the shared expert's output is multiplied by, or nullptr: one
     const T* y;                     // [tokens][width]: its output, or nullptr: the two below
-    const T* down;                  // [width][inter]
+    const T* down;                  // [width][inter], or nullptr (and y nullptr): no shared expert
     const T* hidden;                // [tokens][inter]
     int inter;
 };
@@ -282,7 +299,7 @@ __global__ __launch_bounds__(256) void experts_down_kernel(const T* __restrict__
             if (chosen[(size_t)t * top + s] >= experts) total += weights[(size_t)t * top + s];
         identity_weight = total;
     }
-    const float gate = beside.gate ? beside.gate[t] : 0.f;
+    const float gate = beside.gate ? beside.gate[t] : 1.f;
     const bool shared_vectors = beside.inter % V == 0 && ((reinterpret_cast<size_t>(beside.down) | reinterpret_cast<size_t>(beside.hidden)) & 15) == 0;
     __syncthreads();
     const int c0 = blockIdx.y * columns_per_block, c1 = min(width, c0 + columns_per_block);
@@ -363,7 +380,7 @@ LSA_EXPORT int lsa_route_top(const float* logits, int experts, int top, int* cho
 
 LSA_EXPORT int lsa_experts_gate_up(int code, const void* x, const void* gate_up, const int* chosen, void* hidden, int n, int top,
                                    int inter, int width, int experts, float limit, int identity, const void* shared_gate_up,
-                                   void* shared_hidden, int shared_inter, hipStream_t stream) {
+                                   void* shared_hidden, int shared_inter, int plain, hipStream_t stream) {
     if (n <= 0) return 0;
     if (shared_gate_up != nullptr && (shared_hidden == nullptr || shared_inter < 1)) return -1;
     const int most_inter = shared_gate_up && shared_inter > inter ? shared_inter : inter;
@@ -372,8 +389,8 @@ LSA_EXPORT int lsa_experts_gate_up(int code, const void* x, const void* gate_up,
     if (!in_lds) lds = 0;
     const int columns = 16;
     dim3 grid(n * (top + (shared_gate_up ? 1 : 0)), (most_inter + columns - 1) / columns);
-    if (code) experts_gate_up_kernel<bf16_t><<<grid, 256, lds, stream>>>((const bf16_t*)x, (const bf16_t*)gate_up, chosen, (bf16_t*)hidden, top, inter, width, experts, columns, in_lds, limit, identity, (const bf16_t*)shared_gate_up, (bf16_t*)shared_hidden, shared_inter);
-    else experts_gate_up_kernel<float><<<grid, 256, lds, stream>>>((const float*)x, (const float*)gate_up, chosen, (float*)hidden, top, inter, width, experts, columns, in_lds, limit, identity, (const float*)shared_gate_up, (float*)shared_hidden, shared_inter);
+    if (code) experts_gate_up_kernel<bf16_t><<<grid, 256, lds, stream>>>((const bf16_t*)x, (const bf16_t*)gate_up, chosen, (bf16_t*)hidden, top, inter, width, experts, columns, in_lds, limit, identity, (const bf16_t*)shared_gate_up, (bf16_t*)shared_hidden, shared_inter, plain);
+    else experts_gate_up_kernel<float><<<grid, 256, lds, stream>>>((const float*)x, (const float*)gate_up, chosen, (float*)hidden, top, inter, width, experts, columns, in_lds, limit, identity, (const float*)shared_gate_up, (float*)shared_hidden, shared_inter, plain);
     LSA_LAUNCH_CHECK();
 }
 
@@ -381,7 +398,7 @@ LSA_EXPORT int lsa_experts_down(int code, const void* hidden, const void* down, 
                                 int n, int top, int inter, int width, int experts, const void* x, const float* shared_gate, const void* shared_y,
                                 const void* shared_down, const void* shared_hidden, int shared_inter, hipStream_t stream) {
     if (n <= 0) return 0;
-    if ((shared_gate != nullptr) != (shared_y != nullptr || shared_down != nullptr) || (shared_down != nullptr && shared_hidden == nullptr)) return -1;
+    if ((shared_gate != nullptr && shared_y == nullptr && shared_down == nullptr) || (shared_down != nullptr && shared_hidden == nullptr)) return -1;
     // (a block takes four columns: staging the token's hidden rows in LDS would cost as much as it reads of the weights)
     const size_t lds = 0;
     const bool in_lds = false;
@@ -440,17 +457,19 @@ typedef float f32x4 __attribute__((ext_vector_type(4)));
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 
 // C = A . B^T for one tile of 64 sorted pairs and 128 rows of the expert's matrix (K contiguous in both).
+// FORM 0: the products themselves.  FORM 2: max(product, 0)^2.  FORM 1 is GATED:
 //   GATED: B's 128 rows are 64 gate rows f0 .. f0 + 63 and their 64 up rows; the result is silu(gate) * up, 64 columns.
 //   Rows of A: a[(sorted[i] / pair_div)] (pair_div = top for the tokens' rows, 1 for the pairs' hidden rows).
 // Four wavefronts, each 32 rows x 16 NT columns (GATED: half of them gate columns, half their up columns): 2 x NT MFMA
 // tiles of 16 x 16, k in steps of 32.  A slab of BK columns of K of both operands goes through LDS (rows padded by 16
 // bytes).  NT = 4 where an expert has few pairs (its weights bound the time), 8 where it has many (every operand read
 // from LDS then feeds more products, which is what bounds a tile of 4).
-template <int BK, bool GATED, typename O, int NT>
+template <int BK, int FORM, typename O, int NT>
 __global__ __launch_bounds__(256) void experts_tile_kernel(const bf16_t* __restrict__ a, int a_stride, int pair_div,
                                                            const bf16_t* __restrict__ b, long expert_stride, int b_rows, int b_up_offset,
                                                            const int* __restrict__ sorted, const int* __restrict__ tile_expert,
                                                            O* __restrict__ out, int out_stride, int n_out, int k, float limit) {
+    constexpr bool GATED = FORM == 1;
     constexpr int ROW = BK + 8;                                    // elements of a padded row in LDS
     __shared__ __align__(16) bf16_t a_lds[TILE_M * ROW];
     constexpr int BN = 32 * NT;                                    // rows of B a block takes
@@ -556,7 +575,7 @@ __global__ __launch_bounds__(256) void experts_tile_kernel(const bf16_t* __restr
 #pragma unroll
                 for (int j = 0; j < NT; ++j) {
                     const int c = n0 + wave_n * (BN / 2) + 16 * j + col;
-                    if (c < n_out) o[c] = (O)acc[i][j][r];
+                    if (c < n_out) o[c] = (O)(FORM == 2 ? rectified_square(acc[i][j][r]) : acc[i][j][r]);
                 }
             }
         }
@@ -576,9 +595,9 @@ __global__ __launch_bounds__(256) void experts_combine_kernel(const float* __res
     float acc[V];
 #pragma unroll
     for (int v = 0; v < V; ++v) acc[v] = 0.f;
-    if (beside.gate) {
+    if (beside.y) {
         const Halves h = *reinterpret_cast<const Halves*>(beside.y + (size_t)t * width + c);
-        const float gate = beside.gate[t];
+        const float gate = beside.gate ? beside.gate[t] : 1.f;
 #pragma unroll
         for (int v = 0; v < V; ++v) acc[v] = gate * (float)h.v[v];
     }
@@ -612,9 +631,9 @@ LSA_EXPORT int lsa_experts_tile_rows() { return TILE_M; }
 LSA_EXPORT int lsa_experts_tiled(const void* x, const void* gate_up, const void* down, const int* chosen, const float* weights,
                                  void* hidden, float* y, float* out, int* sorted, int* tile_expert, int max_tiles, int n, int top,
                                  int inter, int width, int experts, float limit, int identity, const float* shared_gate, const void* shared_y,
-                                 hipStream_t stream) {
+                                 int plain, hipStream_t stream) {
     if (n <= 0) return 0;
-    if ((shared_gate != nullptr) != (shared_y != nullptr)) return -1;
+    if (shared_gate != nullptr && shared_y == nullptr) return -1;
     const int pairs = n * top;
     if (width % 32 || inter % 32 || max_tiles < (pairs + TILE_M - 1) / TILE_M + experts || (size_t)experts * 8 > 60000) return -1;
     experts_sort_kernel<<<1, 1024, (size_t)experts * 2 * sizeof(int), stream>>>(chosen, pairs, experts, sorted, tile_expert, max_tiles);
@@ -624,9 +643,10 @@ LSA_EXPORT int lsa_experts_tiled(const void* x, const void* gate_up, const void*
     bf16_t* hb = (bf16_t*)hidden;
     const bool many = pairs >= 16 * experts;                    // pairs to an expert: wide tiles pay
 #define LSA_TILES(BK, NT) do { \
-        dim3 grid1(max_tiles, (inter + 16 * NT - 1) / (16 * NT)), grid2(max_tiles, (width + 32 * NT - 1) / (32 * NT)); \
-        if (!second) experts_tile_kernel<BK, true, bf16_t, NT><<<grid1, 256, 0, stream>>>(xb, width, top, gu, (long)2 * inter * width, 2 * inter, inter, sorted, tile_expert, hb, inter, inter, width, limit); \
-        else experts_tile_kernel<BK, false, float, NT><<<grid2, 256, 0, stream>>>(hb, inter, 1, dn, (long)width * inter, width, 0, sorted, tile_expert, y, width, width, inter, 0.f); \
+        dim3 grid1(max_tiles, (inter + 16 * NT - 1) / (16 * NT)), gridp(max_tiles, (inter + 32 * NT - 1) / (32 * NT)), grid2(max_tiles, (width + 32 * NT - 1) / (32 * NT)); \
+        if (!second && plain) experts_tile_kernel<BK, 2, bf16_t, NT><<<gridp, 256, 0, stream>>>(xb, width, top, gu, (long)inter * width, inter, 0, sorted, tile_expert, hb, inter, inter, width, 0.f); \
+        else if (!second) experts_tile_kernel<BK, 1, bf16_t, NT><<<grid1, 256, 0, stream>>>(xb, width, top, gu, (long)2 * inter * width, 2 * inter, inter, sorted, tile_expert, hb, inter, inter, width, limit); \
+        else experts_tile_kernel<BK, 0, float, NT><<<grid2, 256, 0, stream>>>(hb, inter, 1, dn, (long)width * inter, width, 0, sorted, tile_expert, y, width, width, inter, 0.f); \
     } while (0)
     for (int pass = 0; pass < 2; ++pass) {
         const bool second = pass == 1;

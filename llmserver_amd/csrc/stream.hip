@@ -181,6 +181,72 @@ __global__ __launch_bounds__(256) void scaled_norm_add_kernel(const float* __res
     }
 }
 
+// out = rmsnorm(alpha * x + y) * weight in float32 (out may be x); `rounded` (may be null) gets it as well.  One workgroup a
+// token; a thread issues the loads of its first SUM_CACHE pieces of V numbers (x, y and the weights), none under a condition,
+// before the sum of squares and keeps them; the rest of longer rows is formed again behind it by the thread that owns it.
+constexpr int SUM_CACHE = 4;
+template <typename Y, typename R, int V>
+__global__ __launch_bounds__(256) void sum_norm_kernel(const float* x, const Y* __restrict__ y, float alpha, const float* __restrict__ weight,
+                                                       float eps, float* out, R* __restrict__ rounded, int width) {
+    struct alignas(4 * V) Floats { float v[V]; };
+    struct alignas(sizeof(Y) * V) Ys { Y v[V]; };
+    struct alignas(sizeof(R) * V) Rs { R v[V]; };
+    __shared__ float scratch[16];
+    const size_t base = (size_t)blockIdx.x * width;
+    const int stride = blockDim.x * V;
+    float s[SUM_CACHE][V], w[SUM_CACHE][V];
+#pragma unroll
+    for (int k = 0; k < SUM_CACHE; ++k) {
+        const int i = min((int)threadIdx.x * V + k * stride, width - V);
+        const Floats a = *reinterpret_cast<const Floats*>(x + base + i), b = *reinterpret_cast<const Floats*>(weight + i);
+        const Ys c = *reinterpret_cast<const Ys*>(y + base + i);
+#pragma unroll
+        for (int v = 0; v < V; ++v) {
+            s[k][v] = alpha * a.v[v] + (float)c.v[v];
+            w[k][v] = b.v[v];
+        }
+    }
+    float sq = 0.f;
+#pragma unroll
+    for (int k = 0; k < SUM_CACHE; ++k)
+        if ((int)threadIdx.x * V + k * stride < width)
+#pragma unroll
+            for (int v = 0; v < V; ++v) sq += s[k][v] * s[k][v];
+    for (int i = threadIdx.x * V + SUM_CACHE * stride; i < width; i += stride)
+#pragma unroll
+        for (int v = 0; v < V; ++v) {
+            const float u = alpha * x[base + i + v] + (float)y[base + i + v];
+            sq += u * u;
+        }
+    const float inv = rsqrtf(block_sum(sq, scratch) / (float)width + eps);
+    auto finish = [&](int i, const float (&u)[V], const float (&factor)[V]) {
+        Floats f;
+#pragma unroll
+        for (int v = 0; v < V; ++v) f.v[v] = u[v] * inv * factor[v];
+        *reinterpret_cast<Floats*>(out + base + i) = f;
+        if (rounded) {
+            Rs r;
+#pragma unroll
+            for (int v = 0; v < V; ++v) r.v[v] = (R)f.v[v];
+            *reinterpret_cast<Rs*>(rounded + base + i) = r;
+        }
+    };
+#pragma unroll
+    for (int k = 0; k < SUM_CACHE; ++k) {
+        const int i = threadIdx.x * V + k * stride;
+        if (i < width) finish(i, s[k], w[k]);
+    }
+    for (int i = threadIdx.x * V + SUM_CACHE * stride; i < width; i += stride) {
+        float u[V], factor[V];
+#pragma unroll
+        for (int v = 0; v < V; ++v) {
+            u[v] = alpha * x[base + i + v] + (float)y[base + i + v];
+            factor[v] = weight[i + v];
+        }
+        finish(i, u, factor);
+    }
+}
+
 // out[c][t] = table[ids[t]] * scale, widened to float32, for each of `copies` equal copies (several residual streams start
 // alike); an id outside the table gives a zero row.
 template <typename T>
@@ -563,6 +629,20 @@ LSA_EXPORT int lsa_short_conv_keep(const float* x, float* state, const int* slot
                                    const int* row_ctx, int kept, int rows, int width, hipStream_t stream) {
     if (rows <= 0 || kept <= 0) return 0;
     short_conv_keep_kernel<<<dim3(rows, (width + 255) / 256), 256, 0, stream>>>(x, state, slots, row_start, row_len, row_ctx, kept, width);
+    LSA_LAUNCH_CHECK();
+}
+
+LSA_EXPORT int lsa_sum_norm(const float* x, const void* y, int y_code, float alpha, const float* weight, float eps, float* out, void* rounded,
+                            int rounded_code, int n, int width, hipStream_t stream) {
+    if (n <= 0) return 0;
+#define LSA_LAUNCH_V(Y, R, V) sum_norm_kernel<Y, R, V><<<n, 256, 0, stream>>>(x, (const Y*)y, alpha, weight, eps, out, (R*)rounded, width)
+#define LSA_LAUNCH(Y, R) do { if (width % 4 == 0) LSA_LAUNCH_V(Y, R, 4); else LSA_LAUNCH_V(Y, R, 1); } while (0)
+    if (y_code && rounded_code) LSA_LAUNCH(bf16_t, bf16_t);
+    else if (y_code) LSA_LAUNCH(bf16_t, float);
+    else if (rounded_code) LSA_LAUNCH(float, bf16_t);
+    else LSA_LAUNCH(float, float);
+#undef LSA_LAUNCH
+#undef LSA_LAUNCH_V
     LSA_LAUNCH_CHECK();
 }
 

@@ -57,7 +57,7 @@ def _weights(model) -> Dict[str, Iterable[ParamSpec]]:
 
 
 def cache_bytes(model, rows: Sequence[StepRow], dtype: torch.dtype) -> float:
-    """What the step's rows read of their caches: the keys and values of a row's context (of its window, where the
+    """What the step's rows read of their caches: the keys and values of a row's context (of its window or chunk, where the
     layer has one) for every call of the order that reads a paged cache, the state of a row for every call with one."""
     element = torch.empty((), dtype=dtype).element_size()
     total = 0.0
@@ -65,7 +65,7 @@ def cache_bytes(model, rows: Sequence[StepRow], dtype: torch.dtype) -> float:
         whole = model.blocks[call.block].cache_spec()
         spec, state = paged_part(whole), state_part(whole)
         if spec is not None:
-            keys = sum(min(row.context, spec.window) if spec.window else row.context for row in rows)
+            keys = sum(row.context - spec.first_key(max(row.context - 1, 0)) for row in rows)
             total += 2.0 * spec.n_kv_heads * spec.head_dim * element * keys
         if state is not None:
             total += math.prod(state.shape) * torch.empty((), dtype=getattr(torch, state.dtype)).element_size() * len(rows)

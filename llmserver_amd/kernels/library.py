@@ -24,7 +24,7 @@ _SIGNATURES = {
     "lsa_sample_static_max_rows": [],
     "lsa_sample_static_error": [c_int],
     "lsa_paged_attention": [_P, c_long, _P, _P, _P, _P, c_int, _P, _P, _P, _P, _P, c_int, _P, c_int, c_int, _P, _P, _P, _P, c_int,
-                            c_float, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, _P, _P, c_float, _P, c_int, c_int, c_int, _P, c_float, _P],
+                            c_float, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, _P, _P, c_float, _P, c_int, c_int, c_int, _P, c_float, c_int, _P, _P, c_long, _P],
     "lsa_embedding_wide": [c_int, _P, _P, _P, c_int, c_int, c_int, c_float, c_int, _P],
     "lsa_stream_inject": [_P, c_int, _P, _P, c_float, _P, _P, c_float, _P, c_int, c_int, c_int, c_int, _P],
     "lsa_most_streams": [],
@@ -41,6 +41,11 @@ _SIGNATURES = {
     "lsa_norm_add_norm": [_P, _P, _P, c_int, c_float, c_float, _P, c_float, _P, _P, c_float, _P, c_int, c_int, c_int, _P],
     "lsa_qkv_prepare": [c_int, _P, c_long, _P, _P, _P, c_int, _P, _P, _P, _P, c_float, _P, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
                         _P, c_int, c_int, c_int, c_int, _P],
+    "lsa_sum_norm": [_P, _P, c_int, c_float, _P, c_float, _P, _P, c_int, c_int, c_int, _P],
+    "lsa_compose_most_width": [],
+    "lsa_compose_most_heads": [],
+    "lsa_qkv_compose": [c_int, _P, c_long, _P, c_int, _P, c_long, _P, _P, _P, _P, c_int, _P, _P, c_int, c_float, _P, c_int, c_int, _P, _P, _P, c_int,
+                        c_int, c_int, c_int, c_int, c_int, c_int, _P, c_float, _P, c_long, _P, c_int, _P],
     "lsa_token_shift": [c_int, _P, _P, c_int, _P, c_long, _P, _P, _P, _P, _P, c_int, c_int, c_int, _P],
     "lsa_token_shift_keep": [c_int, _P, _P, c_long, _P, _P, _P, c_int, c_int, _P],
     "lsa_linear_recurrence_most_dim": [],
@@ -68,9 +73,9 @@ _SIGNATURES = {
                           _P, c_long, _P, c_long, c_int, _P, _P, _P, _P, c_int, _P],
     "lsa_delta_conv_keep": [c_int, _P, c_long, _P, c_long, _P, _P, _P, _P, c_int, c_int, c_int, _P],
     "lsa_delta_rule": [_P, _P, _P, c_int, _P, c_long, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, _P],
-    "lsa_experts_gate_up": [c_int, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_float, c_int, _P, _P, c_int, _P],
+    "lsa_experts_gate_up": [c_int, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_float, c_int, _P, _P, c_int, c_int, _P],
     "lsa_experts_tile_rows": [],
-    "lsa_experts_tiled": [_P, _P, _P, _P, _P, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, _P, _P, _P],
+    "lsa_experts_tiled": [_P, _P, _P, _P, _P, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, _P, _P, c_int, _P],
     "lsa_experts_down": [c_int, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, _P, _P, _P, _P, _P, c_int, _P],
     "lsa_attention_workgroup_tiles": [],
     "lsa_attention_tile_page_multiple": [],

@@ -696,7 +696,7 @@ class HipOps(KernelNamespace):
         return dtype == torch.bfloat16 and head_dim % 64 == 0
 
     def paged_attention(self, qkv, out, keys, values, table, row_start, row_len, row_ctx, plan, scale, window, page_size,
-                        n_q, n_kv, head_dim, ctx, decode_fusion=None, sinks=None, softcap=None):
+                        n_q, n_kv, head_dim, ctx, decode_fusion=None, sinks=None, softcap=None, chunk=None, slopes=None, gates=None):
         """Attention of the step's tokens over their requests' pages.
 
         ``qkv [T, (n_q + 2 n_kv) * d]`` holds the normalised, rotated queries in its first
@@ -709,7 +709,9 @@ class HipOps(KernelNamespace):
 
         Without ``decode_fusion``, ``qkv`` may hold the queries alone (``[T, n_q * d]``).  ``sinks [n_q]`` float32: one
         more term ``exp(sinks[head])`` in the denominator of every softmax of that head (no key, no value).  ``softcap``: scaled
-        scores become ``softcap * tanh(score / softcap)`` before the mask.
+        scores become ``softcap * tanh(score / softcap)`` before the mask.  ``chunk``, ``slopes [n_q]`` (float32; with a positive
+        scale, not with ``decode_fusion``), ``gates`` (a view ``[T, n_q]``): see :class:`KernelNamespace`; the gates join where
+        the results are written.
         """
         n = qkv.shape[0]
         if decode_fusion is None and qkv.shape[1] == n_q * head_dim:
@@ -718,6 +720,12 @@ class HipOps(KernelNamespace):
             _check(qkv, "qkv", None, (n, (n_q + 2 * n_kv) * head_dim))
         if sinks is not None:
             _check(sinks, "sinks", torch.float32, (n_q,))
+        if slopes is not None:
+            _check(slopes, "slopes", torch.float32, (n_q,))
+            if decode_fusion is not None or not scale > 0.0:
+                raise ValueError("a bias by distance takes a positive scale and queries that are ready for attention")
+        if gates is not None:
+            self._strided(gates, "gates", n, n_q, qkv.dtype)
         _check(out, "out", qkv.dtype, (n, n_q * head_dim))
         _check(keys, "keys", qkv.dtype)
         _check(values, "values", qkv.dtype)
@@ -786,7 +794,8 @@ class HipOps(KernelNamespace):
             n_merges, n_slots, _ptr(part_acc), _ptr(part_ml), _ptr(tiles), _ptr(tile_slots), n_tiles, float(scale), int(window) if window else 0,
             page_size, n_q, n_kv, gheads, tokens_per_tile, gtiles, fusion_mode, _ptr(q_weight), _ptr(k_weight), float(norm_eps),
             _ptr(cos_sin), int(plan.get("tiles_per_workgroup", 0)), merge_in_workgroup, int(plan.get("tile_halves", 1)), _ptr(sinks),
-            float(softcap) if softcap else 0.0, _stream()), "paged_attention")
+            float(softcap) if softcap else 0.0, int(chunk) if chunk else 0, _ptr(slopes), _ptr(gates), gates.stride(0) if gates is not None else 0,
+            _stream()), "paged_attention")
 
     # -- a residual stream in float32, attention over a latent, routed experts ---------------------------
     # (libraries of their own, loaded at the first call: models that have none of these parts never build them)
@@ -894,6 +903,18 @@ class HipOps(KernelNamespace):
             _ptr(x), _ptr(y), _ptr(y2), _code(y), a, b, _ptr(weight), float(eps), _ptr(out), _ptr(next_weight), float(next_eps),
             _ptr(normed) if next_weight is not None else None, _code(normed) if next_weight is not None else 0, n, width, _stream()),
             "norm_add_norm")
+
+    def sum_norm(self, x, y, alpha, weight, eps, out, rounded=None):
+        n, width = x.shape
+        _check(x, "x", torch.float32)
+        _check(y, "y", None, (n, width))
+        _check(weight, "weight", torch.float32, (width,))
+        _check(out, "out", torch.float32, (n, width))
+        if rounded is not None:
+            _check(rounded, "rounded", None, (n, width))
+        _launched(self._part_library("stream").lsa_sum_norm(
+            _ptr(x), _ptr(y), _code(y), float(alpha), _ptr(weight), float(eps), _ptr(out), _ptr(rounded),
+            _code(rounded) if rounded is not None else 0, n, width, _stream()), "sum_norm")
 
     def norm_rows(self, x, rows, weight, eps, out):
         n_out, width = out.shape
@@ -1063,30 +1084,35 @@ class HipOps(KernelNamespace):
 
     @staticmethod
     def _expert_limit(activation, limit) -> float:
-        """What the experts' kernels take for the activation: 0 for silu(gate) * up, the limit of the clamped form."""
-        if activation == "silu":
+        """What the experts' kernels take for the activation: the limit of the clamped form, 0 for silu(gate) * up and for
+        the square of the rectifier (of experts without a gate)."""
+        if activation in ("silu", "relu2"):
             return 0.0
         if activation != "clamped" or not limit > 0.0:
-            raise ValueError(f"the experts' kernels compute silu, or the clamped form with a positive limit; asked for {activation!r}, {limit}")
+            raise ValueError(f"the experts' kernels compute silu, relu2, or the clamped form with a positive limit; asked for {activation!r}, {limit}")
         return float(limit)
 
     def experts_gate_up(self, x, gate_up, chosen, hidden, activation="silu", limit=0.0, identity=0, shared=None):
         n, width = x.shape
         experts, top, inter = gate_up.shape[0], chosen.shape[1], hidden.shape[1]
+        plain = activation == "relu2"
+        matrices = 1 if plain else 2
+        if plain and identity:
+            raise ValueError("identity experts stand beside gated ones only")
         _check(x, "x")
-        _check(gate_up, "gate_up", x.dtype, (experts, 2 * inter, width))
+        _check(gate_up, "gate_up", x.dtype, (experts, matrices * inter, width))
         _check(chosen, "chosen", torch.int32, (n, top))
         _check(hidden, "hidden", x.dtype, (n * top, inter))
         shared_inter = 0
         if shared is not None:
             shared_inter = shared[1].shape[1]
-            _check(shared[0], "the shared expert's gate_up", x.dtype, (2 * shared_inter, width))
+            _check(shared[0], "the shared expert's gate_up", x.dtype, (matrices * shared_inter, width))
             _check(shared[1], "the shared expert's hidden", x.dtype, (n, shared_inter))
         _launched(self._part_library("experts").lsa_experts_gate_up(_code(x), _ptr(x), _ptr(gate_up), _ptr(chosen), _ptr(hidden), n, top,
                                                                     inter, width, experts, self._expert_limit(activation, limit), int(identity),
                                                                     _ptr(shared[0]) if shared is not None else None,
-                                                                    _ptr(shared[1]) if shared is not None else None, shared_inter, _stream()),
-                  "experts_gate_up")
+                                                                    _ptr(shared[1]) if shared is not None else None, shared_inter,
+                                                                    1 if plain else 0, _stream()), "experts_gate_up")
 
     @staticmethod
     def _check_beside(like, n, width, x, shared_y, shared_gate):
@@ -1106,8 +1132,8 @@ class HipOps(KernelNamespace):
         _check(weights, "weights", torch.float32, (n, top))
         _check(out, "out", torch.float32)
         self._check_beside(hidden, n, width, x, shared_y, shared_gate)
-        if (shared_gate is None) != (shared is None and shared_y is None) or (shared is not None and shared_y is not None):
-            raise ValueError("a shared expert comes with its gate, and as its output or as its matrix and hidden rows")
+        if (shared_gate is not None and shared is None and shared_y is None) or (shared is not None and shared_y is not None):
+            raise ValueError("a shared expert comes as its output or as its matrix and hidden rows, a gate with one of them")
         shared_inter = 0
         if shared is not None:
             shared_inter = shared[1].shape[1]
@@ -1132,8 +1158,9 @@ class HipOps(KernelNamespace):
         experts, top, inter = gate_up.shape[0], chosen.shape[1], down.shape[2]
         if x.dtype != torch.bfloat16 or width % 32 or inter % 32 or n * top <= experts or experts > 4096:
             return False
+        plain = activation == "relu2"
         _check(x, "x")
-        _check(gate_up, "gate_up", x.dtype, (experts, 2 * inter, width))
+        _check(gate_up, "gate_up", x.dtype, (experts, inter if plain else 2 * inter, width))
         _check(down, "down", x.dtype, (experts, width, inter))
         _check(chosen, "chosen", torch.int32, (n, top))
         _check(weights, "weights", torch.float32, (n, top))
@@ -1147,7 +1174,8 @@ class HipOps(KernelNamespace):
         scratch = torch.empty((max_tiles * (tile + 1),), device=x.device, dtype=torch.int32)
         _launched(lib.lsa_experts_tiled(_ptr(x), _ptr(gate_up), _ptr(down), _ptr(chosen), _ptr(weights), _ptr(hidden), _ptr(y), _ptr(out),
                                         _ptr(scratch), scratch[max_tiles * tile:].data_ptr(), max_tiles, n, top, inter, width, experts,
-                                        self._expert_limit(activation, limit), int(identity), _ptr(shared_gate), _ptr(shared_y), _stream()),
+                                        self._expert_limit(activation, limit), int(identity), _ptr(shared_gate), _ptr(shared_y),
+                                        1 if plain else 0, _stream()),
                   "experts_tiled")
         return True
 
@@ -1189,6 +1217,64 @@ class HipOps(KernelNamespace):
             _code(qkv), _ptr(qkv), qkv.shape[1], _ptr(keys), _ptr(values), _ptr(table), table.shape[1], _ptr(token_row), _ptr(positions),
             _ptr(q_weight), _ptr(k_weight), float(eps), _ptr(cos_sin), pairs, page_size, n_q, n_kv, dim, value_dim, row, _ptr(out_q),
             1 if write_cache else 0, n, 1 if pairing == "halves" else 0, int(value_share), _stream()), "qkv_prepare")
+
+    SPANS = (None, "head", "projection")       # what queries and keys are normed over (the kernel's codes)
+
+    def qkv_compose(self, qkv, taps, state, state_slots, token_row, positions, row_start, q_weight, k_weight, span, eps, cos_sin, pairing,
+                    keys, values, table, page_size, n_q, n_kv, dim, value_dim, out_q, mix=0.0, first=None, own_values=None, keep=False):
+        n, rows = qkv.shape[0], row_start.shape[0]
+        q_width, k_width, v_width = n_q * dim, n_kv * dim, n_kv * value_dim
+        channels = q_width + k_width + v_width
+        if keep and n != rows:
+            raise ValueError("the state moves on inside this kernel only in steps of one token per row")
+        if pairing not in ("neighbours", "halves") or span not in self.SPANS:
+            raise ValueError(f"dimensions turn in neighbouring pairs or in halves, norms run over {self.SPANS}; got {pairing!r}, {span!r}")
+        lib = self._part_library("compose")
+        if max(q_width, k_width) > lib.lsa_compose_most_width() or max(n_q, n_kv) > lib.lsa_compose_most_heads():
+            raise ValueError(f"the kernel takes rows of up to {lib.lsa_compose_most_width()} numbers in up to {lib.lsa_compose_most_heads()} heads, "
+                             f"got {n_q} / {n_kv} heads of {dim}")
+        if qkv.dim() != 2 or qkv.shape[1] < channels:
+            raise ValueError(f"qkv must bring at least {channels} columns, it has the shape {tuple(qkv.shape)}")
+        self._strided(qkv, "qkv", n, qkv.shape[1])
+        _code(qkv)
+        pointer, stride, count = None, 0, 0
+        if taps is not None:
+            count = taps.shape[0]
+            _check(taps, "taps", torch.float32, (count, channels))
+            if count > 1:
+                _check(state_slots, "state_slots", torch.int32, (rows,))
+                pointer, stride = self._state_rows(state, 0, (count - 1) * channels, "state")
+        _check(token_row, "token_row", torch.int32, (n,))
+        _check(positions, "positions", torch.int32, (n,))
+        _check(row_start, "row_start", torch.int32)
+        if (q_weight is None) != (k_weight is None) or (q_weight is not None and span is None):
+            raise ValueError("q and k norm weights come together, with a norm")
+        if q_weight is not None:
+            for name, w, width in (("q_weight", q_weight, q_width), ("k_weight", k_weight, k_width)):
+                _check(w, name, torch.float32, (dim if span == "head" else width,))
+        pairs = 0
+        if cos_sin is not None:
+            pairs = cos_sin.shape[1] // 2
+            _check(cos_sin, "cos_sin", torch.float32, (n, 2 * pairs))
+            if 2 * pairs > dim:
+                raise ValueError(f"{2 * pairs} dimensions turn, a head has {dim}")
+        pages, row = keys.shape[0], keys.shape[-1]
+        _check(keys, "keys", qkv.dtype, (pages, n_kv, page_size, row))
+        _check(values, "values", qkv.dtype, (pages, n_kv, row, page_size))
+        if dim > row or value_dim > row or page_size % 4:
+            raise ValueError(f"heads of {dim} / {value_dim} do not fit the pages' rows of {row}, or pages of {page_size} keys are no multiple of 4")
+        _check(table, "table", torch.int32, (rows, table.shape[1]))
+        _check(out_q, "out_q", qkv.dtype, (n, n_q * row))
+        if first is not None:
+            self._strided(first, "first", n, v_width, qkv.dtype)
+        if own_values is not None:
+            _check(own_values, "own_values", qkv.dtype, (n, v_width))
+        _launched(lib.lsa_qkv_compose(
+            _code(qkv), qkv.data_ptr(), qkv.stride(0), _ptr(taps), count, pointer, stride, _ptr(state_slots) if pointer is not None else None,
+            _ptr(token_row), _ptr(positions), _ptr(row_start), 1 if keep else 0, _ptr(q_weight), _ptr(k_weight), self.SPANS.index(span), float(eps),
+            _ptr(cos_sin), pairs, 1 if pairing == "halves" else 0, _ptr(keys), _ptr(values), _ptr(table), table.shape[1], page_size, n_q, n_kv, dim,
+            value_dim, row, _ptr(out_q), float(mix), _ptr(first), first.stride(0) if first is not None else 0, _ptr(own_values), n, _stream()),
+            "qkv_compose")
 
     # -- a block whose sublayers join the stream together; differential attention; the gated delta rule ------------------
     def gated_pair_update(self, x, gates, y1, scale1, y2, scale2, next_weight=None, next_eps=0.0, normed=None):

@@ -1,8 +1,9 @@
-from .attention import AttentionNames, AttentionPlan, AttentionTuning, GQAttention, TileLaunchCost, build_attention_plan, group_tiling
+from .attention import (AttentionNames, AttentionPlan, AttentionTuning, GQAttention, TileLaunchCost, ValueMixing, build_attention_plan,
+                        group_tiling)
 from .base import (INT_TABLE, MATRIX, VECTOR, Block, FeedForward, Mixer, Norm, PagedAndStateSpec, PagedKVSpec, ParamSpec, Part,
                    PositionEncoding, StateSpec)
 from .block import (DepthAverage, HyperConnection, LoopSteps, MultiStreamBlock, ParallelGatedBlock, PassEntry, PostNormBlock, PreNormBlock,
-                    SandwichBlock)
+                    SandwichBlock, SumNormBlock)
 from .conv import ShortConvolution
 from .decayed import Retention, RetentionNames, StateSpaceDuality, StateSpaceNames
 from .delta import GatedDeltaNames, GatedDeltaRule
@@ -27,4 +28,4 @@ __all__ = ["KernelNamespace", "AttentionNames", "AttentionTuning", "TileLaunchCo
            "ScaledPair", "HyperConnection", "MultiStreamBlock", "PlainMLP", "StreamReadNorm", "MatrixMemory", "MatrixMemoryNames",
            "GatedLinearAttention", "GatedLinearAttentionNames", "TimeMixing", "TimeMixingNames", "TokenShift", "ParallelGatedBlock",
            "GatedDeltaRule", "GatedDeltaNames", "DifferentialAttention", "DifferentialNames", "Retention", "RetentionNames",
-           "StateSpaceDuality", "StateSpaceNames", "LoopSteps", "PassEntry", "SharedExpert", "YarnScaling"]
+           "StateSpaceDuality", "StateSpaceNames", "LoopSteps", "PassEntry", "SharedExpert", "YarnScaling", "SumNormBlock", "ValueMixing"]

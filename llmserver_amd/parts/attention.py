@@ -26,7 +26,7 @@ from typing import Optional, Tuple
 import numpy as np
 import torch
 
-from .base import VECTOR, Mixer, PagedKVSpec, ParamSpec, PositionEncoding
+from .base import VECTOR, Mixer, PagedAndStateSpec, PagedKVSpec, ParamSpec, PositionEncoding, StateSpec
 from .kernel_namespace import tuning_of
 from .linear import Linear
 
@@ -98,6 +98,24 @@ class AttentionNames:
     out: str = "o_proj"
     q_norm: str = "q_norm"
     k_norm: str = "k_norm"
+    gate: str = "g_proj"            # a gate of one number a head, where the mixer has one
+    conv_suffix: str = ".conv"      # the taps of a short convolution over time: ``<tensor of qkv><conv_suffix>``
+
+
+@dataclasses.dataclass(frozen=True)
+class ValueMixing:
+    """A layer's values join those that the first layer with this mixing computed for the same token (behind its convolution,
+    if it has one): ``v <- (1 - lambda) v + lambda v_first``, ``lambda`` one number of the checkpoint (``tensor``).  ``first``:
+    this is that layer; its values stay as they are, its number is not used.  ``name`` tells several such chains of layers
+    of a model apart."""
+    first: bool
+    tensor: str = "vmix"
+    name: str = "values"
+
+
+def distance_slopes(heads: int) -> list:
+    """What a head takes off a score per position between query and key: ``2^(-8 (h + 1) / heads)`` for head ``h`` = 0, 1, ..."""
+    return [2.0 ** (-8.0 * (head + 1) / heads) for head in range(heads)]
 
 
 def group_tiling(group_size: int, tile_rows: int = TILE_ROWS):
@@ -153,7 +171,14 @@ def _ranges_of_steps(steps, walk, most_ranges):
     return np.minimum(most_ranges, np.maximum(1, -(-steps // walk)))
 
 
-def _workgroups_of_rows(rows, row_len, row_ctx, tokens_per_tile, window, per_workgroup):
+def first_keys(positions, window: Optional[int], chunk: Optional[int] = None):
+    """The first key that a query at each of ``positions`` (an int64 array) sees: all of them, those of a window, those of
+    the position's own chunk (:class:`~llmserver_amd.parts.base.PagedKVSpec`)."""
+    first = np.zeros_like(positions) if window is None else np.maximum(0, positions - window + 1)
+    return first if chunk is None else np.maximum(first, positions // chunk * chunk)
+
+
+def _workgroups_of_rows(rows, row_len, row_ctx, tokens_per_tile, window, per_workgroup, chunk=None):
     """The workgroups that ``rows`` make with ``per_workgroup`` tiles each, all rows at once: arrays of their row, first
     token, first key, one past the last key, and tiles (the last workgroup of a row may have fewer)."""
     lens = row_len[rows]
@@ -163,14 +188,14 @@ def _workgroups_of_rows(rows, row_len, row_ctx, tokens_per_tile, window, per_wor
     of_row = np.repeat(np.arange(len(rows)), groups_of_row)
     starts = (np.arange(int(groups_of_row.sum())) - np.repeat(np.cumsum(groups_of_row) - groups_of_row, groups_of_row)) * span
     k_end = first_positions[of_row] + np.minimum(starts + span, lens[of_row])
-    k_begin = np.zeros_like(starts) if window is None else np.maximum(0, first_positions[of_row] + starts - window + 1)
+    k_begin = first_keys(first_positions[of_row] + starts, window, chunk)
     tiles = -(-np.minimum(span, lens[of_row] - starts) // tokens_per_tile)
     return rows[of_row], starts, k_begin, k_end, tiles
 
 
 def _workgroup_tiles_that_pay(row_len, row_ctx, tiles_per_row, tokens_per_tile, heads, window, most: int,
                               tuning: AttentionTuning = DEFAULT_TUNING, most_halves: int = 1, most_ranges: int = 1,
-                              min_tiles: int = MIN_TILES_FOR_WORKGROUPS, workgroups: Optional[dict] = None):
+                              min_tiles: int = MIN_TILES_FOR_WORKGROUPS, workgroups: Optional[dict] = None, chunk: Optional[int] = None):
     """``(tiles per workgroup, halves, walk)`` of the prompt-portion kernel that the step's rows finish soonest with:
     4 or ``most`` tiles, the keys of a workgroup walked whole or, where the kernel can, in two halves side by side,
     and, where the kernel can (``most_ranges`` > 1), cut into ranges of at most ``walk`` steps for workgroups of
@@ -187,7 +212,7 @@ def _workgroup_tiles_that_pay(row_len, row_ctx, tiles_per_row, tokens_per_tile, 
     row_len, row_ctx = np.asarray(row_len, dtype=np.int64), np.asarray(row_ctx, dtype=np.int64)
     best, best_key = None, None
     for per_workgroup in sorted({min(4, most), most}):
-        of_rows = _workgroups_of_rows(rows, row_len, row_ctx, tokens_per_tile, window, per_workgroup)
+        of_rows = _workgroups_of_rows(rows, row_len, row_ctx, tokens_per_tile, window, per_workgroup, chunk)
         if workgroups is not None:
             workgroups[per_workgroup] = of_rows                  # (the caller goes on with those of the way chosen)
         _, _, k_begin, k_end, tiles_of_group = of_rows
@@ -223,14 +248,14 @@ SHORT_CONTEXT = 512     # captured steps whose contexts all stay within this are
 
 
 def _single_token_plan(row_ctx: np.ndarray, window: Optional[int], splits: int, merge_in_workgroup: int = 0,
-                       key_align: int = KEY_ALIGN) -> AttentionPlan:
+                       key_align: int = KEY_ALIGN, chunk: Optional[int] = None) -> AttentionPlan:
     """The plan of a step in which every row brings one token and every tile gets ``splits`` key ranges: what the
     loop of :func:`build_attention_plan` makes for it, row by row, computed for all rows at once (a decode step of
     many rows is planned thousands of times a second)."""
     n_rows = len(row_ctx)
     rows = np.arange(n_rows, dtype=np.int64)
     k_end = row_ctx
-    k_begin = np.zeros_like(k_end) if window is None else np.maximum(0, k_end - window)
+    k_begin = first_keys(k_end - 1, window, chunk)
     zeros = np.zeros_like(rows)
     if splits <= 1 and not merge_in_workgroup:
         items = np.stack([rows, zeros, k_begin, k_end], axis=1).astype(np.int32)
@@ -260,8 +285,9 @@ def build_attention_plan(row_len, row_ctx, group_size: int, n_kv_heads: int, win
                          target_waves: int = TARGET_WAVES, fixed_splits: Optional[int] = None,
                          workgroup_tiles: int = 0, single_token_shortcut: bool = True, merge_in_workgroup: int = 0,
                          tuning: AttentionTuning = DEFAULT_TUNING, tile_halves: int = 1, tile_min_workgroups: int = 0,
-                         tile_key_ranges: int = 1, fixed_tiles: Optional[int] = None) -> AttentionPlan:
-    """Cut the step's rows into tiles of tokens and, where that pays, ranges of keys.
+                         tile_key_ranges: int = 1, fixed_tiles: Optional[int] = None, chunk: Optional[int] = None) -> AttentionPlan:
+    """Cut the step's rows into tiles of tokens and, where that pays, ranges of keys.  ``window`` / ``chunk``: which keys a
+    query sees (see :func:`first_keys`); a tile's keys begin at the first one that its first token sees.
 
     With ``fixed_splits`` every tile gets exactly that many items (some may be empty), so the
     arrays have the same shape whatever the contexts are.  With ``workgroup_tiles`` (the number of tiles a
@@ -288,7 +314,7 @@ def build_attention_plan(row_len, row_ctx, group_size: int, n_kv_heads: int, win
     if merge_in_workgroup not in (0, 2, WORKGROUP_RANGES) or (merge_in_workgroup == 2 and len(row_len) % 2):
         raise ValueError("a workgroup merges four key ranges of one tile, or two ranges of each of two tiles (an even number of rows)")
     if (merge_in_workgroup or (single_token_shortcut and fixed_splits is not None)) and single_tokens:
-        return _single_token_plan(row_ctx, window, int(fixed_splits or merge_in_workgroup or 1), merge_in_workgroup, key_align)
+        return _single_token_plan(row_ctx, window, int(fixed_splits or merge_in_workgroup or 1), merge_in_workgroup, key_align, chunk)
     if merge_in_workgroup:
         # Rows of several tokens: every tile of every row gets exactly four ranges (the last ones may be empty), four
         # neighbouring items, which their workgroup merges: no slots, no merge, and no workgroups of tiles.
@@ -306,7 +332,7 @@ def build_attention_plan(row_len, row_ctx, group_size: int, n_kv_heads: int, win
     if workgroup_tiles and fixed_splits is None and int(tiles_per_row[tiles_per_row >= min_tiles].sum()) >= MIN_TILES_FOR_WORKGROUPS:
         per_workgroup, halves, walk = _workgroup_tiles_that_pay(
             row_len, row_ctx, tiles_per_row, tokens_per_tile, n_kv_heads * group_tiles, window, int(workgroup_tiles), tuning,
-            int(tile_halves), most_ranges, min_tiles, workgroups=workgroups)
+            int(tile_halves), most_ranges, min_tiles, workgroups=workgroups, chunk=chunk)
         if per_workgroup and tile_min_workgroups:
             groups = sum(-(-int(n) // (per_workgroup * tokens_per_tile)) for n, tiles_of_row in zip(row_len, tiles_per_row)
                          if tiles_of_row >= min_tiles)
@@ -318,7 +344,7 @@ def build_attention_plan(row_len, row_ctx, group_size: int, n_kv_heads: int, win
         # first + j * ranges + s, where ``first`` is the group's first slot.
         rows_in_tiles = np.flatnonzero(tiles_per_row >= min_tiles)
         of_row, starts, k_begin, k_end, tiles_of_group = workgroups.get(per_workgroup) or _workgroups_of_rows(
-            rows_in_tiles, row_len, row_ctx, tokens_per_tile, window, per_workgroup)
+            rows_in_tiles, row_len, row_ctx, tokens_per_tile, window, per_workgroup, chunk)
         aligned = (k_begin // key_align) * key_align
         steps = -(-(k_end - aligned) // key_step)
         per = -(-steps // _ranges_of_steps(steps, walk, most_ranges)) * key_step
@@ -354,7 +380,7 @@ def build_attention_plan(row_len, row_ctx, group_size: int, n_kv_heads: int, win
         q1 = np.minimum(q0 + tokens_per_tile, row_len[t_row])
         first_pos = (row_ctx - row_len)[t_row]
         t_end = first_pos + q1                           # last query of the tile sees keys < t_end
-        t_begin = np.zeros_like(t_end) if window is None else np.maximum(0, first_pos + q0 - window + 1)
+        t_begin = first_keys(first_pos + q0, window, chunk)
         if fixed_splits is not None:
             splits = np.full(len(t_row), int(fixed_splits), dtype=np.int64)
         elif waves_unsplit < target_waves:
@@ -413,7 +439,8 @@ def build_attention_plan(row_len, row_ctx, group_size: int, n_kv_heads: int, win
     return plan
 
 
-def stage_attention_plan(ctx, key, group_size: int, n_kv_heads: int, head_dim: int, window: Optional[int], graph_shape) -> None:
+def stage_attention_plan(ctx, key, group_size: int, n_kv_heads: int, head_dim: int, window: Optional[int], graph_shape,
+                         chunk: Optional[int] = None) -> None:
     """Make the step's attention work list for a mixer of this geometry and put it among the step's staged arrays under
     ``key`` (mixers of equal geometry share it).  ``graph_shape``: the mixer's :meth:`Mixer.graph_shape`."""
     if ctx.has_plan(key):
@@ -450,7 +477,7 @@ def stage_attention_plan(ctx, key, group_size: int, n_kv_heads: int, head_dim: i
     plan = build_attention_plan(ctx.h_row_len, ctx.h_row_ctx, group_size, n_kv_heads, window,
                                 target_waves=tuning.target_waves, fixed_splits=fixed, workgroup_tiles=per_workgroup,
                                 merge_in_workgroup=in_workgroup, tuning=tuning, tile_halves=halves, tile_min_workgroups=fewest,
-                                tile_key_ranges=key_ranges, fixed_tiles=fixed_tiles)
+                                tile_key_ranges=key_ranges, fixed_tiles=fixed_tiles, chunk=chunk)
     ctx.set_plan(key, {
         **({"tile_slots": plan.tile_slots} if plan.tile_slots is not None else {}),
         "items": plan.items, "item_slot": plan.item_slot, "merges": plan.merges, "tiles": plan.tiles,
@@ -471,7 +498,9 @@ class GQAttention(Mixer):
                  qk_norm_eps: Optional[float] = None, bias: bool = False, out_bias: Optional[bool] = None,
                  window: Optional[int] = None, scale: Optional[float] = None, names: AttentionNames = AttentionNames(),
                  sinks: Optional[str] = None, softcap: Optional[float] = None, value_dim: Optional[int] = None,
-                 bare_names: bool = False, bias_suffix: str = "", values_are_keys: bool = False):
+                 bare_names: bool = False, bias_suffix: str = "", values_are_keys: bool = False,
+                 norm_span: str = "head", norm_weights: bool = True, chunk: Optional[int] = None, distance_bias: bool = False,
+                 conv_taps: int = 0, head_gate: bool = False, value_mixing: Optional[ValueMixing] = None):
         """``sinks``: the checkpoint name of a float vector ``[n_heads]`` whose exponentials join the softmax's
         denominators (one term per head, without a key or a value), or None.  ``softcap``: scores become
         ``softcap * tanh(score / softcap)`` (after the scale, before the mask), or None.  ``value_dim``: the size of a
@@ -480,6 +509,16 @@ class GQAttention(Mixer):
         no value projection; a token's value row is what the key product left (bias included), taken before norm and rotation.
         ``names.qkv`` then names queries and keys only, and the stacked matrix gets the keys' rows a second time in
         the values' place when the tensors have been loaded, so every kernel sees queries, keys and values as usual.
+
+        ``norm_span``: what the query and key norm runs over, a ``"head"`` (one weight for all heads) or the whole
+        ``"projection"`` (a weight per channel of it); ``norm_weights``: False, nothing multiplies the normed rows (the
+        norm over a head without a weight is the same before and behind the rotation, which keeps a head's length).
+        ``chunk``: queries see the keys of their own chunk only (:class:`~llmserver_amd.parts.base.PagedKVSpec`).
+        ``distance_bias``: a score, after scale and cap, loses :func:`distance_slopes` times the positions between query and
+        key.  ``conv_taps``: queries, keys and values each pass a causal convolution over time per channel right behind
+        the product (bias included), tap ``j`` on the token ``conv_taps - 1 - j`` places back, zeros before the sequence; a request
+        keeps the last ``conv_taps - 1`` rows of the product as state.  ``head_gate``: a head's result is multiplied by
+        the sigmoid of one more row a head of the product.  ``value_mixing``: see :class:`ValueMixing`; the mixed values are cached.
 
         A position encoding that turns neighbouring dimensions together (``pairing == "neighbours"``), a rotation of a
         part of the head, values of another size than the keys, and head sizes that are no multiple of 16 go the general
@@ -493,7 +532,18 @@ class GQAttention(Mixer):
         paired = getattr(position, "pairing", None) == "neighbours"
         self.general = paired or self.value_dim != head_dim or head_dim % 16 != 0 or \
             (position.rotary_dim is not None and position.rotary_dim != head_dim)
+        if norm_span not in ("head", "projection"):
+            raise ValueError(f"queries and keys are normed over a head or over the whole projection, not over {norm_span!r}")
+        self.norm_span, self.norm_weights = norm_span, bool(norm_weights)
+        self.chunk = int(chunk) if chunk else None
+        self.distance_bias, self.conv_taps, self.head_gate, self.value_mixing = bool(distance_bias), int(conv_taps), bool(head_gate), value_mixing
+        # queries, keys and values need more than norm and rotation on their way from the product to attention
+        self.composed = self.conv_taps > 0 or value_mixing is not None or norm_span != "head" or not self.norm_weights
+        self.general = self.general or self.composed or self.head_gate
         if self.general:
+            if values_are_keys and self.composed or head_gate and (bias or len(names.qkv) != 3):
+                raise ValueError("keys that serve as values have no convolution, mixing or wider norm of their own; a gate comes beside "
+                                 "three projections without biases")
             if position.rotary_dim is not None and position.rotary_dim > head_dim:
                 raise ValueError(f"the position encoding rotates {position.rotary_dim} dimensions, a head has {head_dim}")
         self.pairing = "neighbours" if paired else "halves"
@@ -513,16 +563,27 @@ class GQAttention(Mixer):
         if len(names.qkv) not in stacked:
             raise ValueError(f"queries, keys and values come in one, two or three checkpoint tensors, not {len(names.qkv)}")
         self.names, self.bare_names = names, bare_names
-        self.qkv = Linear(width, names.qkv, stacked[len(names.qkv)], bias, bare_names=bare_names, bias_suffix=bias_suffix)
+        pieces, sizes = tuple(names.qkv), stacked[len(names.qkv)]
+        if head_gate:
+            pieces, sizes = (*pieces, names.gate), (*sizes, n_heads)
+        self.channels = q_rows + k_rows + v_rows                # ... of the product, in front of the gates
+        self.qkv = Linear(width, pieces, sizes, bias, bare_names=bare_names, bias_suffix=bias_suffix)
         self.o = Linear(n_heads * self.value_dim, (names.out,), (width,), bias if out_bias is None else out_bias, bare_names=bare_names,
                         bias_suffix=bias_suffix)
         self.q_norm_weight = None
         self.k_norm_weight = None
         self.sinks_name, self.sinks = sinks, None
         self._o_padded = None
+        self._taps = {}
+        self.conv_weight = None         # float32 [taps, channels]
+        self.slopes = None              # float32 [n_heads]
+        self.mix = 0.0                  # the layer's lambda, a number
 
     def cache_spec(self):
-        return PagedKVSpec(self.n_kv_heads, self.row, self.window)
+        paged = PagedKVSpec(self.n_kv_heads, self.row, self.window, self.chunk)
+        if self.conv_taps < 2:
+            return paged
+        return PagedAndStateSpec(paged, StateSpec((-(-(self.conv_taps - 1) * self.channels // 4) * 4,), "float32"))
 
     def _norm_names(self):
         suffix = "" if self.bare_names else ".weight"
@@ -530,9 +591,14 @@ class GQAttention(Mixer):
 
     def param_specs(self):
         specs = {**self.qkv.param_specs(), **self.o.param_specs()}
-        if self.qk_norm_eps is not None:
-            for name in self._norm_names():
-                specs[name] = ParamSpec((self.head_dim,), VECTOR, "norm")
+        if self.qk_norm_eps is not None and self.norm_weights:
+            for name, heads in zip(self._norm_names(), (self.n_heads, self.n_kv_heads)):
+                specs[name] = ParamSpec((self.head_dim if self.norm_span == "head" else heads * self.head_dim,), VECTOR, "norm")
+        if self.conv_taps:
+            for name, size in zip(self.names.qkv, self.qkv.piece_out):
+                specs[name + self.names.conv_suffix] = ParamSpec((size, self.conv_taps), VECTOR, "normal")
+        if self.value_mixing is not None:
+            specs[self.value_mixing.tensor] = ParamSpec((), VECTOR, "bias", optional=self.value_mixing.first)
         if self.sinks_name is not None:
             specs[self.sinks_name] = ParamSpec((self.n_heads,), VECTOR, "normal")
         return specs
@@ -541,6 +607,10 @@ class GQAttention(Mixer):
         owner = name if self.bare_names else name.rsplit(".", 1)[0]
         if name == self.sinks_name:
             self.sinks = tensor
+        elif self.conv_taps and name.endswith(self.names.conv_suffix) and name[:-len(self.names.conv_suffix)] in self.names.qkv:
+            self._taps[name[:-len(self.names.conv_suffix)]] = tensor
+        elif self.value_mixing is not None and name == self.value_mixing.tensor:
+            self.mix = float(tensor)
         elif owner == self.names.q_norm:
             self.q_norm_weight = tensor
         elif owner == self.names.k_norm:
@@ -555,6 +625,15 @@ class GQAttention(Mixer):
     def finalize(self):
         self.qkv.finalize()
         self.o.finalize()
+        if self.conv_taps:
+            self.conv_weight = torch.cat([self._taps[name] for name in self.names.qkv], dim=0).t().contiguous()
+            self._taps.clear()
+        if self.distance_bias:
+            self.slopes = torch.tensor(distance_slopes(self.n_heads), dtype=torch.float32, device=self.qkv.weight.device)
+        if self.head_gate and self.qkv.weight.shape[0] % 8:
+            # rows of zeros behind the gates, so that every token's row of the product begins at a multiple of 16 bytes
+            weight = self.qkv.weight
+            self.qkv.weight = torch.cat([weight, weight.new_zeros((-weight.shape[0] % 8, weight.shape[1]))], dim=0).contiguous()
         if self.values_are_keys and self.qkv.weight.shape[0] == (self.n_heads + self.n_kv_heads) * self.head_dim:
             # the keys' rows once more, where the kernels look for the values
             from_keys = self.n_heads * self.head_dim
@@ -573,7 +652,7 @@ class GQAttention(Mixer):
             self._o_padded = padded.view(weight.shape[0], self.n_heads * self.row).contiguous()
 
     def plan_key(self):
-        return ("paged_attention", self.group_size, self.n_kv_heads, self.window, self.row)
+        return ("paged_attention", self.group_size, self.n_kv_heads, self.window, self.row) + ((self.chunk,) if self.chunk else ())
 
     def graph_shape(self, rows: int, longest_context: int):
         return "short contexts" if longest_context <= SHORT_CONTEXT else None
@@ -584,14 +663,43 @@ class GQAttention(Mixer):
     def mixing_flops(self, new_tokens: int, context: int) -> float:
         """Scores and weighted values: two products of ``head_dim`` multiply-adds per query head, query and visible key."""
         first = context - new_tokens
-        if self.window is None:
+        if self.chunk is not None:
+            spec = PagedKVSpec(self.n_kv_heads, self.row, self.window, self.chunk)
+            pairs = sum(position + 1 - spec.first_key(position) for position in range(first, context))
+        elif self.window is None:
             pairs = new_tokens * first + new_tokens * (new_tokens + 1) // 2
         else:
             pairs = sum(min(position + 1, self.window) for position in range(first, context))
         return 2.0 * self.n_heads * (self.head_dim + self.value_dim) * pairs
 
     def prepare(self, ctx):
-        stage_attention_plan(ctx, self.plan_key(), self.group_size, self.n_kv_heads, self.row, self.window, self.graph_shape)
+        stage_attention_plan(ctx, self.plan_key(), self.group_size, self.n_kv_heads, self.row, self.window, self.graph_shape, self.chunk)
+
+    def _compose(self, qkv, ctx, cache, table, q):
+        """Convolution, norm and rotation of queries and keys, convolution and mixing of values, and the cache write."""
+        values, own, first = {}, None, None
+        width = self.n_kv_heads * self.value_dim
+        if self.value_mixing is not None:
+            key = ("first values", self.value_mixing.name)
+            if self.value_mixing.first:
+                # (without a convolution the product's own columns are the values)
+                own = ctx.empty((qkv.shape[0], width)) if self.conv_taps else None
+                kept = own if own is not None else qkv[:, self.channels - width:self.channels]
+                ctx.computed(key, lambda: kept)
+            else:
+                first = ctx.computed(key, lambda: None)
+                if first is None or first.shape[1] != width:
+                    raise ValueError("values are mixed with those of an earlier layer that has as many of them")
+                values = {"mix": self.mix, "first": first}
+        single = ctx.n_tokens == ctx.n_rows         # one token a row: the thread that reads a row's last inputs also moves them on
+        state = cache.state if self.conv_taps > 1 else None
+        ctx.ops.qkv_compose(qkv, self.conv_weight, state, ctx.state_slots, ctx.token_row, ctx.positions, ctx.row_start, self.q_norm_weight,
+                            self.k_norm_weight, self.norm_span if self.qk_norm_eps is not None else None,
+                            self.qk_norm_eps if self.qk_norm_eps is not None else 0.0, self.position.cos_sin(ctx), self.pairing,
+                            cache.keys, cache.values, table, cache.page_size, self.n_heads, self.n_kv_heads, self.head_dim, self.value_dim,
+                            q, own_values=own, keep=single and state is not None, **values)
+        if state is not None and not single:
+            ctx.ops.delta_conv_keep(qkv, self.channels, self.conv_taps, state, 0, ctx.state_slots, ctx.row_start, ctx.row_len, ctx.row_ctx)
 
     def _forward_general(self, x, ctx, cache, sink):
         """Norm, rotation of neighbouring pairs, rows filled up to the kernels' head size: a kernel in front of attention."""
@@ -599,22 +707,34 @@ class GQAttention(Mixer):
         table = ctx.block_table(cache.group)
         n = qkv.shape[0]
         q = ctx.empty((n, self.n_heads * self.row))
-        ctx.ops.qkv_prepare(qkv, cache.keys, cache.values, table, ctx.token_row, ctx.positions, self.q_norm_weight, self.k_norm_weight,
-                            self.qk_norm_eps if self.qk_norm_eps is not None else 0.0, self.position.cos_sin(ctx), cache.page_size,
-                            self.n_heads, self.n_kv_heads, self.head_dim, self.value_dim, q, cache.writable,
-                            **({"pairing": "halves"} if self.pairing == "halves" and self.position.rotary_dim is not None else {}))
+        if self.composed or self.head_gate:
+            if not cache.writable:
+                raise ValueError("this mixer writes the pages it reads")
+            self._compose(qkv, ctx, cache, table, q)
+        else:
+            ctx.ops.qkv_prepare(qkv, cache.keys, cache.values, table, ctx.token_row, ctx.positions, self.q_norm_weight, self.k_norm_weight,
+                                self.qk_norm_eps if self.qk_norm_eps is not None else 0.0, self.position.cos_sin(ctx), cache.page_size,
+                                self.n_heads, self.n_kv_heads, self.head_dim, self.value_dim, q, cache.writable,
+                                **({"pairing": "halves"} if self.pairing == "halves" and self.position.rotary_dim is not None else {}))
         out = ctx.empty((n, self.n_heads * self.row))
         extra = {}
         if self.sinks is not None:
             extra["sinks"] = self.sinks
         if self.softcap is not None:
             extra["softcap"] = self.softcap
+        if self.head_gate:
+            extra["gates"] = qkv[:, self.channels:self.channels + self.n_heads]
+        extra.update(self._seen())
         ctx.ops.paged_attention(q, out, cache.keys, cache.values, table, ctx.row_start, ctx.row_len, ctx.row_ctx,
                                 ctx.get_plan(self.plan_key()), self.scale, self.window, cache.page_size,
                                 self.n_heads, self.n_kv_heads, self.row, ctx, **extra)
         if self._o_padded is None:
             return self.o.forward(out, ctx, sink=sink)
         return ctx.ops.linear(out, self._o_padded)
+
+    def _seen(self):
+        """What the attention kernels are told of scores and keys beyond scale, cap and window."""
+        return {**({"chunk": self.chunk} if self.chunk else {}), **({"slopes": self.slopes} if self.slopes is not None else {})}
 
     def forward(self, x, ctx, cache, sink=None):
         if self.general:
@@ -640,6 +760,7 @@ class GQAttention(Mixer):
             extra["sinks"] = self.sinks
         if self.softcap is not None:
             extra["softcap"] = self.softcap
+        extra.update(self._seen())
         ctx.ops.paged_attention(
             qkv, out, cache.keys, cache.values, table, ctx.row_start, ctx.row_len, ctx.row_ctx,
             ctx.get_plan(self.plan_key()), self.scale, self.window, cache.page_size,

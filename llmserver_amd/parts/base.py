@@ -43,10 +43,27 @@ class ParamSpec:
 @dataclasses.dataclass(frozen=True)
 class PagedKVSpec:
     """Keys and values of every token, in pages.  ``window`` None keeps all keys; a number keeps
-    only the last ``window`` keys a query can see, so earlier pages can be given back."""
+    only the last ``window`` keys a query can see, so earlier pages can be given back.  ``chunk``: a query sees the keys of
+    its own chunk only, chunks of that many positions counted from the sequence's first one (None: no chunks); the pages
+    of a chunk can be given back when the next one begins."""
     n_kv_heads: int
     head_dim: int
     window: Optional[int] = None
+    chunk: Optional[int] = None
+
+    @property
+    def bounded(self) -> bool:
+        """Whether queries stop seeing keys as a sequence goes on."""
+        return self.window is not None or self.chunk is not None
+
+    def first_key(self, position: int) -> int:
+        """The first position that a query at ``position`` sees."""
+        first = 0
+        if self.window is not None:
+            first = max(first, position - self.window + 1)
+        if self.chunk is not None:
+            first = max(first, position // self.chunk * self.chunk)
+        return first
 
 
 @dataclasses.dataclass(frozen=True)
@@ -120,7 +137,8 @@ class StreamUpdate:
     """What a part may return instead of a plain update of the residual stream, when its last
     projection has already added the update and prepared the norm that follows.
 
-    ``resid [T, H]`` is the stream with the update added, ``norm`` the norm that was prepared, in one of two ways.
+    ``resid [T, H]`` is the stream with the update added, ``norm`` the norm that was prepared (None: the stream itself,
+    rounded to the compute type, for a block whose sublayers read it unnormed), in one of two ways.
     Either ``weighted [T, H] = resid * norm.weight`` and ``square_sums [T, P]``, float32 partial sums of
     ``resid^2`` over P parts of each row: a projection that reads ``weighted`` and divides its result rows by
     ``sqrt(sum(square_sums) / H + eps)`` has multiplied the normalised stream.  Or ``normed [T, H]``, the norm's

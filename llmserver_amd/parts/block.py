@@ -183,6 +183,64 @@ class PostNormBlock(Block):
         return result, None
 
 
+class SumNormBlock(Block):
+    """Sublayers that read the stream itself; the norm stands behind the sum: ``x <- n1(alpha * x + mixer(x))``, then
+    ``x <- n2(alpha * x + ffn(x))``, the stream in 32-bit throughout; ``ffn`` may be None.  The scaled sum, the norm and the
+    rounded copy that the next sublayer reads are one kernel (``ops.sum_norm``)."""
+
+    def __init__(self, mixer: Mixer, mixer_norm: Norm, ffn=None, ffn_norm=None, alpha: float = 1.0,
+                 names=("mix", "norm1", "mlp", "norm2")):
+        self.mixer, self.mixer_norm, self.ffn, self.ffn_norm, self.alpha = mixer, mixer_norm, ffn, ffn_norm, float(alpha)
+        self.names = tuple(names)
+
+    def _parts(self):
+        parts = dict(zip(self.names[:2], (self.mixer, self.mixer_norm)))
+        if self.ffn is not None:
+            parts.update(zip(self.names[2:], (self.ffn, self.ffn_norm)))
+        return parts
+
+    def param_specs(self):
+        return {f"{prefix}.{name}" if name else prefix: spec for prefix, part in self._parts().items()
+                for name, spec in part.param_specs().items()}
+
+    def assign(self, name, tensor):
+        parts = self._parts()
+        if name in parts:                                   # the part's name is the tensor's
+            parts[name].assign("", tensor)
+            return
+        prefix, rest = name.split(".", 1)
+        parts[prefix].assign(rest, tensor)
+
+    def finalize(self):
+        for part in self._parts().values():
+            part.finalize()
+
+    def _behind(self, x, result, norm, ctx):
+        """``(stream, rows that the next sublayer reads)`` behind a sublayer; the stream is updated where it lies."""
+        rounded = None if ctx.dtype == torch.float32 else ctx.empty(x.shape)
+        ctx.ops.sum_norm(x, result, self.alpha, norm.weight, norm.eps, x, rounded=rounded)
+        return x, x if rounded is None else rounded
+
+    def forward(self, resid, delta, ctx, cache):
+        """``delta``: None, or a :class:`StreamUpdate` without a norm whose ``normed`` rows are the stream in the compute type."""
+        x, h = resid, None
+        if isinstance(delta, StreamUpdate):
+            x = delta.resid
+            h = delta.normed if delta.norm is None else None
+        elif delta is not None:
+            raise ValueError("this block takes a stream to which everything has been added")
+        if h is None:
+            h = x if ctx.dtype == torch.float32 else x.to(ctx.dtype)
+        x, h = self._behind(x, self.mixer.forward(h, ctx, cache), self.mixer_norm, ctx)
+        if self.ffn is not None:
+            if getattr(self.ffn, "reads_stream", False):
+                fed = self.ffn.forward(h, ctx, stream=x)
+            else:
+                fed = self.ffn.forward(h, ctx)
+            x, h = self._behind(x, fed, self.ffn_norm, ctx)
+        return x, StreamUpdate(None, x, normed=h)
+
+
 class SandwichBlock(Block):
     """A norm in front of every sublayer and one behind it: ``x <- x + n1b(mixer(n1(x)))``, then
     ``x <- x + n2b(ffn(n2(x)))``, the stream in 32-bit throughout; ``ffn`` may be None.  The norm behind a sublayer, the

@@ -5,7 +5,8 @@ ones) and weighted by the softmax over the chosen logits only.  ``scoring="sigmo
 ``groups=(count, keep)`` the experts form ``count`` equal groups of neighbours, a group's score is the sum of its two
 largest scores, and only experts of the ``keep`` best groups can be chosen; the ``top`` largest scores are chosen and
 are the weights as they are.  Expert: ``D (act(G h) * (U h))`` with ``act = silu``, or, with ``activation="clamped"``,
-``g = min(G h, limit)``, ``u = clamp(U h, -limit, limit)``, ``D (g * sigmoid(1.702 g) * (u + 1))``; no biases.
+``g = min(G h, limit)``, ``u = clamp(U h, -limit, limit)``, ``D (g * sigmoid(1.702 g) * (u + 1))``; with ``activation="relu2"``
+there is no gate: ``D max(U h, 0)^2``; no biases.
 ``scoring="softmax_all"``: scores are the softmax over all experts; the ``top`` largest of score + a correction per expert are
 chosen; their scores, divided by their sum (+ 1e-20) and times a constant, are the weights.
 
@@ -18,7 +19,7 @@ the list of chosen experts on the device: nothing of the routing is read on the 
 from __future__ import annotations
 
 import dataclasses
-from typing import Tuple
+from typing import Optional, Tuple
 
 import torch
 
@@ -28,18 +29,20 @@ from .linear import Linear
 
 @dataclasses.dataclass(frozen=True)
 class SharedExpert:
-    """A gated feed-forward of its own inner size that every token uses; names below ``prefix``."""
+    """A feed-forward of the routed experts' form and of its own inner size that every token uses; names below ``prefix``
+    (``pieces``: as the routed experts')."""
     intermediate: int
     prefix: str = "shared"
-    pieces: Tuple[str, str, str] = ("gate", "up", "down")
-    gate: str = "sg"            # the row [1, W] whose product's sigmoid multiplies the result
+    pieces: Tuple[str, ...] = ("gate", "up", "down")
+    gate: Optional[str] = "sg"      # the row [1, W] whose product's sigmoid multiplies the result (None: nothing does)
 
 
 class RoutedExperts(FeedForward):
     reads_stream = True       # forward takes ``stream=``: the 32-bit rows that ``x`` was rounded from, for the router
 
     SCORINGS = ("softmax", "sigmoid", "softmax_all")
-    ACTIVATIONS = ("silu", "clamped")
+    ACTIVATIONS = ("silu", "clamped", "relu2")
+    UNGATED = ("relu2",)            # experts of two matrices: ``pieces`` names the up and the down matrix
 
     def __init__(self, width: int, intermediate: int, experts: int, top: int, router: str = "router", expert: str = "e{}",
                  pieces=("gate", "up", "down"), scoring: str = "softmax", groups=None, activation: str = "silu", limit: float = 0.0,
@@ -57,8 +60,11 @@ class RoutedExperts(FeedForward):
             count, keep = groups
             if scoring != "sigmoid" or experts % count or not 1 <= keep <= count or top > keep * (experts // count):
                 raise ValueError(f"{experts} experts in {count} groups of which {keep} are kept, {top} chosen, scoring {scoring!r}")
-        if shared is not None and activation != "silu":
-            raise ValueError("the shared expert's activation is silu; so has to be the routed experts'")
+        if shared is not None and activation == "clamped":
+            raise ValueError("the shared expert's activation is silu or the square of the rectifier, as the routed experts' then is")
+        self.gated = activation not in self.UNGATED
+        if any(len(names) != (3 if self.gated else 2) for names in (pieces, *((shared.pieces,) if shared is not None else ()))):
+            raise ValueError(f"an expert with the activation {activation!r} has {3 if self.gated else 2} matrices, named are {tuple(pieces)}")
         if activation == "clamped" and not limit > 0.0:
             raise ValueError("the clamped activation needs its limit")
         self.scoring, self.groups, self.activation, self.limit = scoring, tuple(groups) if groups is not None else None, activation, float(limit)
@@ -75,18 +81,18 @@ class RoutedExperts(FeedForward):
         self.shared_gate = None
         self.shared_gate_up = self.shared_down = None
         if shared is not None:
-            gate, up, down = (f"{shared.prefix}.{piece}" for piece in shared.pieces)
-            self.shared_gate_name = f"{shared.prefix}.{shared.gate}"
-            self.shared_gate_up = Linear(width, (gate, up), (shared.intermediate, shared.intermediate), bare_names=True)
+            *ups, down = (f"{shared.prefix}.{piece}" for piece in shared.pieces)
+            self.shared_gate_name = f"{shared.prefix}.{shared.gate}" if shared.gate is not None else None
+            self.shared_gate_up = Linear(width, ups, (shared.intermediate,) * len(ups), bare_names=True)
             self.shared_down = Linear(shared.intermediate, (down,), (width,), bare_names=True)
-        self.gate_up = None       # [experts, 2F, W]
+        self.gate_up = None       # [experts, 2F, W]; without gates [experts, F, W]
         self.down = None          # [experts, W, F]
 
     def _names(self):
-        gate, up, down = self.pieces
+        """(names of the matrices that read the token, name of the one that writes) of every expert."""
         for index in range(self.experts):
-            prefix = self.expert_name.format(index)
-            yield index, f"{prefix}.{gate}", f"{prefix}.{up}", f"{prefix}.{down}"
+            *ups, down = (f"{self.expert_name.format(index)}.{piece}" for piece in self.pieces)
+            yield ups, down
 
     def param_specs(self):
         share = self.top / self.choices
@@ -97,10 +103,11 @@ class RoutedExperts(FeedForward):
             specs[self.correction_name] = ParamSpec((self.choices,), VECTOR, "bias")
         if self.shared is not None:
             specs.update({**self.shared_gate_up.param_specs(), **self.shared_down.param_specs()})
-            specs[self.shared_gate_name] = ParamSpec((1, self.width), VECTOR, "normal")
-        for _, gate, up, down in self._names():
-            specs[gate] = ParamSpec((self.intermediate, self.width), share_per_token=share)
-            specs[up] = ParamSpec((self.intermediate, self.width), share_per_token=share)
+            if self.shared_gate_name is not None:
+                specs[self.shared_gate_name] = ParamSpec((1, self.width), VECTOR, "normal")
+        for ups, down in self._names():
+            for up in ups:
+                specs[up] = ParamSpec((self.intermediate, self.width), share_per_token=share)
             specs[down] = ParamSpec((self.width, self.intermediate), share_per_token=share)
         return specs
 
@@ -111,7 +118,7 @@ class RoutedExperts(FeedForward):
             self.router_bias = tensor
         elif name == self.correction_name:
             self.correction = tensor
-        elif self.shared is not None and name == self.shared_gate_name:
+        elif self.shared is not None and self.shared_gate_name is not None and name == self.shared_gate_name:
             self.shared_gate = tensor
         elif self.shared is not None and self.shared_gate_up.owns(name):
             self.shared_gate_up.assign(name, tensor)
@@ -122,14 +129,15 @@ class RoutedExperts(FeedForward):
 
     def finalize(self):
         names = list(self._names())
-        self.gate_up = torch.stack([torch.cat([self._parts[gate], self._parts[up]], dim=0) for _, gate, up, _ in names]).contiguous()
-        self.down = torch.stack([self._parts[down] for _, _, _, down in names]).contiguous()
+        self.gate_up = torch.stack([torch.cat([self._parts[up] for up in ups], dim=0) for ups, _ in names]).contiguous()
+        self.down = torch.stack([self._parts[down] for _, down in names]).contiguous()
         self._parts.clear()
         if self.shared is not None:
             self.shared_gate_up.finalize()
             self.shared_down.finalize()
-            self.router = torch.cat([self.router, self.shared_gate], dim=0).contiguous()
-            self.shared_gate = None
+            if self.shared_gate is not None:
+                self.router = torch.cat([self.router, self.shared_gate], dim=0).contiguous()
+                self.shared_gate = None
 
     def forward(self, x, ctx, stream=None):
         """``x [T, W]`` in the compute type -> float32 ``[T, W]``.  ``stream``: the same rows in 32-bit, if the caller
@@ -144,7 +152,7 @@ class RoutedExperts(FeedForward):
         if self.scoring == "softmax_all":
             extra.update(correction=self.correction, weight_scale=self.weight_scale)
         shared_gate = None
-        if self.shared is not None:
+        if self.shared is not None and self.shared.gate is not None:
             shared_gate = extra["gate_out"] = ctx.empty((n,), dtype=torch.float32)
         ops.route_experts(x if stream is None else stream, self.router, self.top, chosen, weights, **extra)
         out = ctx.empty((n, self.width), dtype=torch.float32)
@@ -168,7 +176,9 @@ class RoutedExperts(FeedForward):
         return out
 
     def _shared_hidden(self, x, ctx):
-        """The shared expert's ``act(G h) * (U h)`` as products of its own."""
+        """The shared expert's ``act(G h) * (U h)`` (or ``act(U h)``) as products of its own."""
+        if not self.gated:
+            return ctx.ops.linear_activated(x, self.shared_gate_up.weight, self.activation)
         hidden = ctx.ops.linear_gated(x, self.shared_gate_up.weight)
         if hidden is None:
             gate_up = self.shared_gate_up.forward(x, ctx)

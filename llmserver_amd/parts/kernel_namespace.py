@@ -46,10 +46,26 @@ class KernelNamespace:
         raise NotImplementedError
 
     def paged_attention(self, qkv, out, keys, values, table, row_start, row_len, row_ctx, plan, scale, window, page_size,
-                        n_q, n_kv, head_dim, ctx, decode_fusion=None, sinks=None, softcap=None):
+                        n_q, n_kv, head_dim, ctx, decode_fusion=None, sinks=None, softcap=None, chunk=None, slopes=None, gates=None):
         """``sinks [n_q]`` (float32) or None: one more term ``exp(sinks[head])`` in every softmax's denominator, with no
         key and no value.  ``softcap`` (a number or None): scaled scores become ``softcap * tanh(score / softcap)`` before
-        the mask.  ``qkv`` may hold the queries only (``[T, n_q * head_dim]``) where nothing is fused."""
+        the mask.  ``qkv`` may hold the queries only (``[T, n_q * head_dim]``) where nothing is fused.  ``chunk`` (a number or
+        None): a query sees keys of its own chunk only, chunks of so many positions counted from 0.  ``slopes [n_q]`` (float32)
+        or None: a score, after scale and cap, loses ``slopes[head]`` times the positions between query and key.  ``gates``
+        (a view ``[T, n_q]`` of ``qkv``'s type) or None: a head's result is multiplied by the sigmoid of its gate."""
+        raise NotImplementedError
+
+    def qkv_compose(self, qkv, taps, state, state_slots, token_row, positions, row_start, q_weight, k_weight, span, eps, cos_sin, pairing,
+                    keys, values, table, page_size, n_q, n_kv, dim, value_dim, out_q, mix=0.0, first=None, own_values=None, keep=False):
+        """``qkv [T, >= C]`` holds queries ``[n_q * dim]``, keys ``[n_kv * dim]`` and values ``[n_kv * value_dim]``, ``C`` channels.
+        ``taps [K, C]`` (float32) or None: every channel passes a causal convolution over its request's tokens, tap ``j`` on
+        the token ``K - 1 - j`` places back, zeros before the sequence, earlier steps' rows from ``state[slot]`` as ``[K - 1,
+        C]``, oldest first.  Queries and keys are then RMS-normed over each ``"head"`` or over the whole ``"projection"``
+        (``span``; None: no norm), times ``q_weight`` / ``k_weight`` (float32, as long as the span; None: 1), and turned by
+        ``cos_sin`` and ``pairing`` as :meth:`qkv_prepare` turns them; ``out_q`` and the pages' keys get them as there.
+        Values, with ``first`` (a view ``[T, n_kv * value_dim]``): ``(1 - mix) v + mix first``; the pages get them.
+        ``own_values [T, n_kv * value_dim]`` gets the values before the mixing.  ``keep`` (steps of one token per row
+        only): the state also moves on by the step's token, as :meth:`delta_conv_keep` would do."""
         raise NotImplementedError
 
     def qkv_prepare(self, qkv, keys, values, table, token_row, positions, q_weight, k_weight, eps, cos_sin, page_size,
@@ -278,6 +294,11 @@ class KernelNamespace:
         raise NotImplementedError
 
     # Routed experts.
+    def sum_norm(self, x, y, alpha, weight, eps, out, rounded=None):
+        """``out = rmsnorm(alpha * x + y) * weight`` in float32 (``out`` may be ``x``), ``y`` of any type; ``rounded`` (any type)
+        also gets it."""
+        raise NotImplementedError
+
     def route_experts(self, x, router, top, chosen, weights, scoring="softmax", groups=None, bias=None, correction=None, weight_scale=1.0,
                       gate_out=None):
         """Float32 logits ``x router^T``; ``chosen [T, top]`` the largest (first of equals), ``weights`` their softmax.
@@ -292,14 +313,15 @@ class KernelNamespace:
     def experts_gate_up(self, x, gate_up, chosen, hidden, activation="silu", limit=0.0, identity=0, shared=None):
         """``hidden[t * top + s] = silu(G x_t) * (U x_t)`` with ``[G; U] = gate_up[chosen[t, s]]`` (``[E, 2F, W]``);
         ``activation="clamped"``: ``g = min(G x, limit)``, ``u = clamp(U x, -limit, limit)``, ``g * sigmoid(1.702 g) * (u + 1)``.
+        ``activation="relu2"``: experts without a gate, ``gate_up [E, F, W]`` are their up matrices, ``max(U x, 0)^2``.
         ``identity``: that many choices from ``E`` on are identity experts, with nothing to multiply.  ``shared = (gate_up [2F', W],
         hidden [T, F'])``: the shared expert's hidden rows are made beside the others."""
         raise NotImplementedError
 
     def experts_down(self, hidden, down, chosen, weights, out, x=None, shared=None, shared_y=None, shared_gate=None):
         """``out[t] = sum_s weights[t, s] * down[chosen[t, s]] hidden[t * top + s]``; ``down [E, W, F]``, ``out`` float32.
-        ``x [T, W]`` given: choices from ``E`` on are identity experts, whose output is ``x[t]``.  ``shared_gate [T]``: the shared
-        expert's output, ``shared_y [T, W]`` or ``shared = (down [W, F'], hidden [T, F'])``, joins times the gate."""
+        ``x [T, W]`` given: choices from ``E`` on are identity experts, whose output is ``x[t]``.  The shared expert's output,
+        ``shared_y [T, W]`` or ``shared = (down [W, F'], hidden [T, F'])``, joins times ``shared_gate [T]`` (None: 1)."""
         raise NotImplementedError
 
     def sample(self, logits, temperature, uniform, out):

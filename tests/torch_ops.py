@@ -148,7 +148,7 @@ class TorchOps(KernelNamespace):
         values[pages, :, :, slots] = heads[:, n_q + n_kv:].to(values.dtype)
 
     def paged_attention(self, qkv, out, keys, values, table, row_start, row_len, row_ctx, plan, scale, window, page_size,
-                        n_q, n_kv, head_dim, ctx, decode_fusion=None, sinks=None, softcap=None):
+                        n_q, n_kv, head_dim, ctx, decode_fusion=None, sinks=None, softcap=None, chunk=None, slopes=None, gates=None):
         """Per request row: gather its keys/values through the block table, one softmax over all
         keys a query may see (no tiles, no splits).  ``decode_fusion``: the step's rows bring one token each and
         ``qkv`` is the raw projection, which is left as it is."""
@@ -168,6 +168,8 @@ class TorchOps(KernelNamespace):
         for row in range(table.shape[0]):
             start, length, ctx_len = int(row_start[row]), int(row_len[row]), int(row_ctx[row])
             first = 0 if not window else max(0, ctx_len - length - window + 1)
+            if chunk:                                            # (pages of chunks that have ended may be someone else's)
+                first = max(first, (ctx_len - length) // chunk * chunk)
             place = torch.arange(first, ctx_len, device=qkv.device)
             pages = table[row].long()[place // page_size]
             k = keys[pages, :, place % page_size, :].float()            # [keys, n_kv, d]
@@ -182,6 +184,10 @@ class TorchOps(KernelNamespace):
             hidden = place[None, :] > q_pos[:, None]
             if window:
                 hidden = hidden | (place[None, :] <= q_pos[:, None] - window)
+            if chunk:
+                hidden = hidden | (place[None, :] // chunk != q_pos[:, None] // chunk)
+            if slopes is not None:
+                scores = scores - slopes[:, None, None] * (q_pos[:, None] - place[None, :]).float()[None]
             scores = scores.masked_fill(hidden[None], float("-inf"))
             if sinks is None:
                 weights = torch.softmax(scores, dim=-1)
@@ -190,6 +196,8 @@ class TorchOps(KernelNamespace):
                 weights = torch.exp(scores - top[..., None])
                 weights = weights / (weights.sum(dim=-1) + torch.exp(sinks.float()[:, None] - top))[..., None]
             result = torch.einsum("hqk,khd->qhd", weights, v)
+            if gates is not None:
+                result = result * torch.sigmoid(gates[start:start + length].float())[:, :, None]
             out[start:start + length] = result.reshape(length, n_q * head_dim).to(out.dtype)
 
     # -- a 32-bit residual stream -----------------------------------------------------------------------
@@ -231,6 +239,11 @@ class TorchOps(KernelNamespace):
     def norm_rows(self, x, rows, weight, eps, out):
         picked = x if rows is None else x[rows.long()]
         out.copy_((self._rms(picked.float(), eps) * weight).to(out.dtype))
+
+    def sum_norm(self, x, y, alpha, weight, eps, out, rounded=None):
+        out.copy_(self._rms(alpha * x + y.float(), eps) * weight)
+        if rounded is not None:
+            rounded.copy_(out.to(rounded.dtype))
 
     def short_conv(self, x, weight, state, state_slots, token_row, positions, row_start, out, keep=False):
         taps = weight.shape[1]
@@ -317,6 +330,43 @@ class TorchOps(KernelNamespace):
         value_rows[..., :value_dim] = v
         keys[pages, :, slots, :] = key_rows.to(keys.dtype)
         values[pages, :, :, slots] = value_rows.to(values.dtype)
+
+    def qkv_compose(self, qkv, taps, state, state_slots, token_row, positions, row_start, q_weight, k_weight, span, eps, cos_sin, pairing,
+                    keys, values, table, page_size, n_q, n_kv, dim, value_dim, out_q, mix=0.0, first=None, own_values=None, keep=False):
+        n, width, kv = qkv.shape[0], n_kv * value_dim, n_kv * dim
+        channels = n_q * dim + kv + width
+        rows = qkv[:, :channels].float()
+        if taps is not None:
+            count = taps.shape[0]
+            own, rows = rows, torch.zeros_like(rows)
+            for t in range(n):
+                row, position = int(token_row[t]), int(positions[t])
+                begin = position - (t - int(row_start[row]))             # position of the row's first token in this step
+                for j in range(count):
+                    place = position - (count - 1 - j)
+                    if place >= begin:
+                        rows[t] += taps[j] * own[t - (position - place)]
+                    elif place >= 0:
+                        rows[t] += taps[j] * state[int(state_slots[row]), :(count - 1) * channels].view(count - 1, channels)[count - 1 - (begin - place)]
+            if keep:
+                assert n == len(row_start)
+                for t in range(n):
+                    kept = state[int(state_slots[int(token_row[t])])][:(count - 1) * channels]
+                    kept.copy_(torch.cat([kept[channels:], own[t]]))
+        q, k, v = rows[:, :n_q * dim], rows[:, n_q * dim:n_q * dim + kv], rows[:, n_q * dim + kv:]
+        if span == "projection":
+            q, k = self._rms(q, eps), self._rms(k, eps)
+            if q_weight is not None:
+                q, k = q * q_weight, k * k_weight
+        elif span == "head" and q_weight is None:
+            q_weight = k_weight = torch.ones(dim)
+        if own_values is not None:
+            own_values.copy_(v.to(own_values.dtype))
+        if first is not None:
+            v = (1.0 - mix) * v + mix * first.float()
+        weights = (q_weight, k_weight) if span == "head" else (None, None)
+        self.qkv_prepare(torch.cat([q, k, v], dim=1), keys, values, table, token_row, positions, *weights, eps, cos_sin, page_size, n_q, n_kv,
+                         dim, value_dim, out_q, pairing=pairing)
 
     # -- recurrent mixers --------------------------------------------------------------------------------
     def token_shift(self, h, mu, state, offset, state_slots, token_row, positions, row_start, out, keep=False):
@@ -694,6 +744,13 @@ class TorchOps(KernelNamespace):
 
     def experts_gate_up(self, x, gate_up, chosen, hidden, activation="silu", limit=0.0, identity=0, shared=None):
         top, inter = chosen.shape[1], hidden.shape[1]
+        if activation == "relu2":
+            if shared is not None:
+                shared[1].copy_(self.linear_activated(x, shared[0], activation))
+            for t in range(x.shape[0]):
+                for s in range(top):
+                    hidden[t * top + s] = (torch.relu(gate_up[int(chosen[t, s])].float() @ x[t].float()) ** 2).to(hidden.dtype)
+            return
         if shared is not None:
             both = x.float() @ shared[0].float().t()
             gate, up = both[:, :both.shape[1] // 2], both[:, both.shape[1] // 2:]
@@ -716,8 +773,8 @@ class TorchOps(KernelNamespace):
         out.zero_()
         if shared is not None:
             shared_y = shared[1].float() @ shared[0].float().t()
-        if shared_gate is not None:
-            out += shared_gate[:, None] * shared_y.float()
+        if shared_y is not None:
+            out += (1.0 if shared_gate is None else shared_gate[:, None]) * shared_y.float()
         for t in range(out.shape[0]):
             for s in range(top):
                 if x is not None and int(chosen[t, s]) >= down.shape[0]:
