@@ -154,6 +154,27 @@ NAMED_SIZES.update({
 })
 
 
+def _mefurax(width, layers, heads, kv_heads, dim, window, chunk, ff, expert_ff, experts, top, shared, vocab=32768):
+    common = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "v_mix": True}
+    sloped = ("attention", {**common, "conv": 4, "mask": {"size": window}})
+    chunked = ("attention_2", {**common, "mask": {"size": chunk}, "rot": {"base": 10000.0, "dims": dim // 2}, "softcap": 50.0})
+    dense = {"kind": "dense", "ff": ff}
+    moe = {"kind": "moe", "expert": {"ff": expert_ff}, "router": {"experts": experts, "top": top}, "shared": {"ff": shared}}
+    four = [(chunked, dense), (sloped, moe), (chunked, moe), (sloped, moe)]
+    return {"architecture": "Mefurax", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "postln_alpha": 2.0,
+            "layers": [{"type": kind, "mixer": dict(mixer), "mlp": dict(mlp)} for (kind, mixer), mlp in (four * (-(-layers // 4)))[:layers]]}
+
+
+# Mefurax at the widths of the sizes above: 16 (32) heads of 128 over 8 key/value heads in every layer, in turn under chunks of
+# 1,024 positions (rotated, capped, gated) and under a window of 1,024 keys (convolved, normed as a whole, sloped); every layer's
+# values are mixed with the first one's; one layer in four is dense, as large as the dense decoders', the others route: their
+# experts have no gates and as many weights each as those of the Zepolix sizes, and a shared one beside them.
+NAMED_SIZES.update({
+    "mefurax-2k": _mefurax(2048, 8, 16, 8, 128, 1024, 1024, 6 * 1408, 3 * 704, 64, 6, 3 * 704),
+    "mefurax-4k": _mefurax(4096, 8, 32, 8, 128, 1024, 1024, 4 * 2048, 3 * 1024, 32, 4, 3 * 1024),
+})
+
+
 def named_size(name: str) -> dict:
     """The entry's keys, a copy the caller may change (fewer layers, say)."""
     try:

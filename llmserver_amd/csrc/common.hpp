@@ -62,7 +62,7 @@ __device__ inline float block_sum(float v, float* scratch) {
 // Puts 64 consecutive tokens of one KV head, staged in LDS as [VT_TOKENS][pitch] with `filled` numbers a token, into their
 // pages values[page][kv_head][:][slot], zeros for the dimensions from `filled` to d.  Four slots of one dimension go out at
 // a time (8 or 16 bytes) where four tokens are neighbours in one page, which is the rule inside a portion; a page's
-// [d][page_size] block is contiguous, so these stores coalesce.  256 threads; whoever wrote the tile need not have waited.
+// [d][page_size] block is contiguous, so these stores coalesce.  At least 64 threads; whoever wrote the tile need not have waited.
 constexpr int VT_TOKENS = 64;
 template <typename T>
 __device__ __forceinline__ void store_value_tile(const T* tile, int pitch, int token0, int kv_head, int filled, T* __restrict__ values,
@@ -91,7 +91,7 @@ __device__ __forceinline__ void store_value_tile(const T* tile, int pitch, int t
         group_base[threadIdx.x] = base;
     }
     __syncthreads();
-    for (int e = threadIdx.x; e < (VT_TOKENS / 4) * d; e += 256) {
+    for (int e = threadIdx.x; e < (VT_TOKENS / 4) * d; e += blockDim.x) {
         const int g = e & (VT_TOKENS / 4 - 1), i = e / (VT_TOKENS / 4);      // neighbouring threads: neighbouring groups of slots
         const long base = group_base[g];
         if (base < 0) continue;
@@ -102,7 +102,7 @@ __device__ __forceinline__ void store_value_tile(const T* tile, int pitch, int t
         if (sizeof(T) == 2) *reinterpret_cast<uint2*>(dst) = *reinterpret_cast<const uint2*>(four);
         else *reinterpret_cast<uint4*>(dst) = *reinterpret_cast<const uint4*>(four);
     }
-    for (int e = threadIdx.x; e < VT_TOKENS * d; e += 256) {                  // the tokens that are in no such group
+    for (int e = threadIdx.x; e < VT_TOKENS * d; e += blockDim.x) {                  // the tokens that are in no such group
         const int t = e & (VT_TOKENS - 1), i = e / VT_TOKENS;
         const int token = token0 + t;
         if (covered[t] || token >= n_tokens) continue;

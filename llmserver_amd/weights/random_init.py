@@ -88,6 +88,8 @@ def random_model_on_device(config: ModelConfig, device, dtype: torch.dtype, init
         if name in ignored:
             continue
         values = random_tensor(name, spec, init, device=device)
+        if spec.role != INT_TABLE:
+            values = values.to(torch.bfloat16)          # as a model folder would hold them
         model.assign(name, values.to(stored_dtype(spec.role, dtype)))
         assigned.append(name)
         del values

@@ -359,7 +359,7 @@ class TorchOps(KernelNamespace):
             if q_weight is not None:
                 q, k = q * q_weight, k * k_weight
         elif span == "head" and q_weight is None:
-            q_weight = k_weight = torch.ones(dim)
+            q_weight = k_weight = torch.ones(dim, device=qkv.device)
         if own_values is not None:
             own_values.copy_(v.to(own_values.dtype))
         if first is not None:
