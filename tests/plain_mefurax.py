@@ -160,6 +160,11 @@ def expert(h, t, p, r=same):
     return r(relu_squared(h @ t[p + "up"].T)) @ t[p + "down"].T
 
 
+def shared_expert(h, t, p, r=same):
+    """The same; a 16-bit run makes it of products of its own, each of whose results it rounds."""
+    return r(r(relu_squared(r(h @ t[p + "up"].T))) @ t[p + "down"].T)
+
+
 def route(h, t, p, router):
     """(chosen [T, top], weights [T, top]): the largest logits, weighted by the softmax over the chosen ones."""
     picked, chosen = torch.topk(h @ t[p + "router"].T, router["top"], dim=-1)
@@ -175,7 +180,7 @@ def experts(h, read, t, p, mlp, r=same):
         if len(token):
             out[token] += weights[token, place][:, None] * expert(read[token], t, f"{p}e{e}.", r)
     if mlp.get("shared"):
-        out = out + expert(read, t, p + "shared.", r)
+        out = out + shared_expert(read, t, p + "shared.", r)
     return out
 
 
